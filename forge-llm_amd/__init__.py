@@ -15,6 +15,7 @@ LIB_PATH = os.path.join(_HERE, "libforge_hip.so")
 
 Q4_0 = 2
 Q8_0 = 8
+F32, BF16 = 0, 30     # dense model folders (HipModel.from_folder)
 Q4_K, Q6_K = 12, 14   # op level only: ops.QWeight + ops.matmul_vec_q
 FLAG_EXACT = 1   # config.flags / op flags: order-faithful f32 arithmetic (bit-identical to the CPU path)
 FLAG_QKV_BIAS = 2   # config.flags: q, k, v projections add a bias vector before RoPE (Qwen2); the blob carries the vectors
@@ -42,6 +43,8 @@ EXPORTS = [
     "forge_hip_gguf_find_tensor", "forge_hip_gguf_meta", "forge_hip_gguf_config", "forge_hip_gguf_export_weights",
     "forge_hip_gguf_config_mixed", "forge_hip_gguf_export_weights_mixed", "forge_hip_quantize_kquant",
     "forge_hip_model_create_from_gguf", "forge_hip_dequant_ggml", "forge_hip_model_set_repeat_penalty", "forge_hip_apply_repeat_penalty", "forge_hip_sample",
+    "forge_hip_prefill_logits", "forge_hip_model_create_from_folder", "forge_hip_folder_config", "forge_hip_model_config",
+    "forge_hip_model_layer_runs", "forge_hip_prefill_residuals",
 ]
 
 
@@ -95,6 +98,18 @@ def lib():
     L.forge_hip_forward_greedy.argtypes = [vp, u32, C.POINTER(u32)]
     L.forge_hip_prefill_batch.restype = i32
     L.forge_hip_prefill_batch.argtypes = [vp, vp, u64, vp]
+    L.forge_hip_prefill_logits.restype = i32
+    L.forge_hip_prefill_logits.argtypes = [vp, vp, u64, vp, u64, vp]
+    L.forge_hip_prefill_residuals.restype = i32
+    L.forge_hip_prefill_residuals.argtypes = [vp, vp, u64, vp]
+    L.forge_hip_model_layer_runs.restype = u32
+    L.forge_hip_model_layer_runs.argtypes = [vp]
+    L.forge_hip_model_config.restype = i32
+    L.forge_hip_model_config.argtypes = [vp, C.POINTER(Config)]
+    L.forge_hip_folder_config.restype = i32
+    L.forge_hip_folder_config.argtypes = [C.c_char_p, C.POINTER(Config)]
+    L.forge_hip_model_create_from_folder.restype = i32
+    L.forge_hip_model_create_from_folder.argtypes = [C.c_char_p, u32, u32, u32, C.POINTER(vp)]
     L.forge_hip_forward_profile.restype = i32
     L.forge_hip_forward_profile.argtypes = [vp, u32, vp, vp]
     L.forge_hip_prefill_profile.restype = i32

@@ -11,7 +11,11 @@ BUILD = os.path.join(HERE, "build")
 LIB = os.path.join(HERE, "libforge_hip.so")
 
 SOURCES = ["format.hip", "elementwise.hip", "gemv.hip", "gemv_f32.hip", "gemv_kquant.hip", "kquant_prefill.hip", "gemm.hip", "attn_decode.hip", "attn_prefill.hip",
-           "attn_exact.hip", "decode_persistent.hip", "api.hip", "model.hip", "gguf.cpp", "sampling.cpp"]
+           "attn_exact.hip", "decode_persistent.hip", "api.hip", "model.hip", "llama.hip", "block_model.hip", "dense.hip", "attn_latent.hip", "checkpoint.cpp", "gguf.cpp", "sampling.cpp"]
+
+# The trace replay program holds the dense networks only.
+TRACE_RUN = os.path.join(BUILD, "trace_run")
+TRACE_SOURCES = ["format.hip", "elementwise.hip", "model.hip", "block_model.hip", "dense.hip", "attn_latent.hip", "checkpoint.cpp", "trace_run.cpp"]
 
 # -packed-fp32-ops off: keep hipcc from forming packed FP32 instructions.
 # -ffp-contract=off: the CPU path never fuses a*b+c; kernels say fmaf() where a fused op is meant.
@@ -29,7 +33,8 @@ def _hipcc():
 
 def _compile(src):
     obj = os.path.join(BUILD, os.path.splitext(src)[0] + ".o")
-    cmd = [_hipcc(), *FLAGS, "-c", os.path.join(CSRC, src), "-o", obj]
+    part = "%s.%d" % (obj, os.getpid())
+    cmd = [_hipcc(), *FLAGS, "-c", os.path.join(CSRC, src), "-o", part]
     r = subprocess.run(cmd, capture_output=True, text=True)
     # the host pass warns that it does not know the packed-fp32 feature: harmless, filter it
     err = "\n".join(l for l in r.stderr.splitlines() if "packed-fp32-ops" not in l)
@@ -37,20 +42,50 @@ def _compile(src):
         raise RuntimeError(f"hipcc failed on {src}:\n{err}")
     if err.strip():
         sys.stderr.write(err + "\n")
+    os.replace(part, obj)
     return obj
 
 
-def build(verbose=True):
-    os.makedirs(BUILD, exist_ok=True)
-    with ThreadPoolExecutor(max_workers=min(8, len(SOURCES))) as ex:
-        objs = list(ex.map(_compile, SOURCES))
-    cmd = [_hipcc(), "--offload-arch=gfx950", "-shared", "-fPIC", "-o", LIB, *objs]
-    r = subprocess.run(cmd, capture_output=True, text=True)
+def _link(out, objs, *flags):
+    part = "%s.%d" % (out, os.getpid())
+    r = subprocess.run([_hipcc(), "--offload-arch=gfx950", *flags, "-o", part, *objs], capture_output=True, text=True)
     if r.returncode != 0:
         raise RuntimeError("link failed:\n" + r.stderr)
+    os.replace(part, out)
+
+
+def _compile_all(sources):
+    os.makedirs(BUILD, exist_ok=True)
+    with ThreadPoolExecutor(max_workers=min(8, len(sources))) as ex:
+        return list(ex.map(_compile, sources))
+
+
+def build(verbose=True):
+    objs = _compile_all(SOURCES + ["trace_run.cpp"])
+    _link(LIB, objs[:-1], "-shared", "-fPIC")
+    by_name = dict(zip(SOURCES + ["trace_run.cpp"], objs))
+    _link(TRACE_RUN, [by_name[s] for s in TRACE_SOURCES])
     if verbose:
         print(f"built {LIB}")
     return LIB
+
+
+def _older(path, than):
+    return not os.path.exists(path) or os.path.getmtime(path) < than
+
+
+def build_trace_run():
+    """The trace replay program, compiled if it is not there or older than its sources."""
+    headers = [os.path.join(d, f) for d in (CSRC, INCLUDE) for f in os.listdir(d) if f.endswith(".h")] + [os.path.abspath(__file__)]
+    newest_header = max(os.path.getmtime(h) for h in headers)
+    newest = max([newest_header] + [os.path.getmtime(os.path.join(CSRC, s)) for s in TRACE_SOURCES])
+    if _older(TRACE_RUN, newest):
+        obj = lambda s: os.path.join(BUILD, os.path.splitext(s)[0] + ".o")
+        stale = [s for s in TRACE_SOURCES if _older(obj(s), max(newest_header, os.path.getmtime(os.path.join(CSRC, s))))]
+        if stale:
+            _compile_all(stale)
+        _link(TRACE_RUN, [obj(s) for s in TRACE_SOURCES])
+    return TRACE_RUN
 
 
 if __name__ == "__main__":

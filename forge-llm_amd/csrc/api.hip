@@ -1,4 +1,4 @@
-// extern "C" surface, part 1: error string, host format helpers and the op-level entry points.
+// extern "C" surface, part 1: host format helpers and the op-level entry points.
 // The op-level calls own one lazily grown device scratch area per process (activation
 // codes, split-attention partials, rope tables); they are for one caller thread at a time.
 #include <math.h>
@@ -97,14 +97,6 @@ struct forge_hip_qweight {
 };
 
 extern "C" {
-
-const char* forge_hip_last_error(void) { return last_error_cstr(); }
-
-int32_t forge_hip_device_count(void) {
-    int n = 0;
-    if (hipGetDeviceCount(&n) != hipSuccess) return 0;
-    return n;
-}
 
 float forge_hip_f16_to_f32(uint16_t bits) { return f16_to_f32_host(bits); }
 uint16_t forge_hip_f32_to_f16(float x) { return f32_to_f16_host(x); }

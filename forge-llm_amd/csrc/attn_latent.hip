@@ -1,0 +1,573 @@
+// Latent attention: per position the cache holds one latent vector c (RMS-normed) and one rotated key part that all heads share;
+// a head's unrotated key and its value are W_uk c and W_uv c.  An optional window keeps the last `window` positions visible.
+//
+// Prompt rows work on expanded keys and values (a product of the cached latents with [W_uk; W_uv] ahead of the kernel): per
+// (query, key) pair that is dim + rot + vdim multiply-adds against 2 rank + rot on the latents.  Decode works on the latents
+// themselves: the query goes through W_uk^T once, every head then attends to the same cached row, which is read once for 16
+// heads, and the weighted latents go through W_uv once.
+//
+// T: __bf16 or float (dense.h); scores, softmax and sums are 32-bit in both.
+#include <hip/hip_runtime.h>
+
+#include "common.h"
+#include "dense.h"
+#include "dense_gemv.h"
+#include "device_utils.h"
+
+namespace fh {
+
+constexpr float LOG2E = 1.4426950408889634f;
+constexpr uint32_t RANK_MAX = 1024, HEAD_DIM_MAX = 256, SPLITS_MAX = 32;
+
+// ---- the new cache row and the normed query latent of one position; `tid` of `nt` threads, red: LDS, nt / 64 floats -----------------
+__device__ __forceinline__ float block_sum(float v, float* red, uint32_t tid, uint32_t nt) {
+    v = wave_sum(v);
+    __syncthreads();
+    if ((tid & 63) == 0) red[tid >> 6] = v;
+    __syncthreads();
+    float s = 0.f;
+    for (uint32_t i = 0; i < nt / 64; i++) s += red[i];
+    return s;
+}
+
+template <typename T>
+__device__ __forceinline__ void store_cache_row(const LatentShape& sh, const float* raw, const float* kv_norm, const float* cos_t, const float* sin_t,
+                                                uint32_t pos, T* cache, float* red, uint32_t tid, uint32_t nt) {
+    const float* c = raw + sh.q_rank;
+    const float* kr = c + sh.rank;
+    float ss = 0.f;
+    for (uint32_t i = tid; i < sh.rank; i += nt) ss = fmaf(c[i], c[i], ss);      // padding is zero
+    const float inv = 1.0f / sqrtf(block_sum(ss, red, tid, nt) / (float)sh.rank_n + sh.eps);
+    T* row = cache + (size_t)pos * sh.cache_row();
+    for (uint32_t i = tid; i < sh.rank; i += nt) row[i] = (T)(c[i] * inv * kv_norm[i]);
+    for (uint32_t i = tid; i < sh.rot / 2; i += nt) {
+        float u = kr[2 * i], v = kr[2 * i + 1];
+        if (i < sh.rot_pairs) {
+            const float cs = cos_t[(size_t)pos * sh.rot_pairs + i], sn = sin_t[(size_t)pos * sh.rot_pairs + i];
+            const float u2 = u * cs - v * sn;
+            v = v * cs + u * sn;
+            u = u2;
+        }
+        row[sh.rank + 2 * i] = (T)u;
+        row[sh.rank + 2 * i + 1] = (T)v;
+    }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void latent_norm_store_kernel(LatentShape sh, const float* __restrict__ raw, const float* __restrict__ q_norm,
+                                                                const float* __restrict__ kv_norm, const float* __restrict__ cos_t,
+                                                                const float* __restrict__ sin_t, uint32_t base_pos, T* __restrict__ cq, T* __restrict__ cache) {
+    __shared__ float red[4];
+    const uint32_t m = blockIdx.x, tid = threadIdx.x;
+    const float* row = raw + (size_t)m * sh.raw_row();
+    float ss = 0.f;
+    for (uint32_t i = tid; i < sh.q_rank; i += 256) ss = fmaf(row[i], row[i], ss);
+    const float inv = 1.0f / sqrtf(block_sum(ss, red, tid, 256) / (float)sh.q_rank_n + sh.eps);
+    for (uint32_t i = tid; i < sh.q_rank; i += 256) cq[(size_t)m * sh.q_rank + i] = (T)(row[i] * inv * q_norm[i]);
+    store_cache_row<T>(sh, row, kv_norm, cos_t, sin_t, base_pos + m, cache, red, tid, 256);
+}
+
+// ---- prompt ---------------------------------------------------------------------------------------------------------------
+// Workgroup = 4 waves = 128 consecutive queries of one head, 32 per wave; keys and values stream through LDS in tiles of 64
+// (K row-major: unrotated part, rotated part; V transposed), the next tile's loads in registers while this one is worked.  Both
+// products are computed transposed (S^T = K Q^T, O^T = V^T P^T): a lane owns one query, so the softmax statistics are per-lane
+// scalars, and the exponentiated scores are already the second product's operand.  Scores stay in the base-2 domain.
+// DQ >= dim + rot and DV >= vdim: the register tiles' sizes; columns past the real ones are zero.
+template <typename T, int DQ, int DV>
+__global__ __launch_bounds__(256) void latent_attn_prefill_kernel(LatentShape sh, const T* __restrict__ q, const T* __restrict__ kbuf, const T* __restrict__ vbuf,
+                                                                  const T* __restrict__ cache, uint32_t kv_lo, const T* __restrict__ gate, T* __restrict__ out,
+                                                                  uint32_t ld_out, uint32_t M, uint32_t base_pos) {
+    typedef typename Vec<T>::x4 x4;
+    typedef typename Vec<T>::x8 x8;
+    constexpr uint32_t KT = 64, QB = 128, PAD = 16 / sizeof(T);
+    constexpr uint32_t KS = DQ + PAD, VS = KT + 8 / sizeof(T);         // LDS row strides
+    constexpr uint32_t NS = DQ / 16, ND = DV / 32;
+    constexpr uint32_t KP = KT * DQ / 8 / 256, VP = (KT / 2) * (DV / 4) / 256;
+    static_assert(KT * DQ / 8 % 256 == 0 && (KT / 2) * (DV / 4) % 256 == 0, "whole pieces per thread");
+    extern __shared__ __attribute__((aligned(16))) uint8_t lat_lds[];
+    T* Ks = reinterpret_cast<T*>(lat_lds);
+    T* Vt = Ks + KT * KS;
+
+    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, lq = lane & 31, lh = lane >> 5;
+    // latest (longest) query tiles first
+    const uint32_t head = blockIdx.x % sh.heads, ntq = gridDim.x / sh.heads;
+    const uint32_t q0 = (ntq - 1 - blockIdx.x / sh.heads) * QB;
+    const uint32_t dq = sh.dim + sh.rot, window = sh.window ? sh.window : 0xFFFFFFFFu;
+    const float c2 = sh.scale * LOG2E;
+    const uint32_t qrow = q0 + wave * 32 + lq, qpos = base_pos + qrow;
+
+    x8 qf[NS];
+#pragma unroll
+    for (uint32_t s = 0; s < NS; s++) {
+        const uint32_t d = 16 * s + 8 * lh;
+        qf[s] = (qrow < M && d < dq) ? load8(q + (size_t)qrow * sh.q_row() + head * dq + d) : zero8<T>();
+    }
+    v16f oacc[ND];
+#pragma unroll
+    for (uint32_t d = 0; d < ND; d++)
+#pragma unroll
+        for (int r = 0; r < 16; r++) oacc[d][r] = 0.f;
+    float m_run = -INFINITY, l_run = 0.f;
+
+    const uint32_t total = base_pos + M;
+    const uint32_t wg_max = base_pos + min(q0 + QB, M) - 1, wg_min = base_pos + q0;
+    const bool wave_active = q0 + wave * 32 < M;
+    const uint32_t wave_min = wg_min + wave * 32, wave_max = base_pos + min(q0 + wave * 32 + 32, M) - 1;
+    auto first_visible = [&](uint32_t p) { return p >= window ? p - window + 1 : 0u; };
+    const uint32_t wave_lo = first_visible(wave_min);
+    const uint32_t tile0 = first_visible(wg_min) / KT, ntiles = wg_max / KT + 1;
+
+    const uint32_t kst = sh.heads * sh.dim, vst = sh.heads * sh.vdim, cst = sh.cache_row();
+    x8 kreg[KP];
+    x4 va[VP], vb[VP];
+    auto load_tile = [&](uint32_t kt) {
+#pragma unroll
+        for (uint32_t i = 0; i < KP; i++) {
+            const uint32_t idx = tid + 256 * i, key = idx / (DQ / 8), d = idx % (DQ / 8) * 8, t = kt * KT + key;
+            if (t >= total || d >= dq) kreg[i] = zero8<T>();
+            else kreg[i] = d < sh.dim ? load8(kbuf + (size_t)(t - kv_lo) * kst + head * sh.dim + d)
+                                      : load8(cache + (size_t)t * cst + sh.rank + (d - sh.dim));
+        }
+#pragma unroll
+        for (uint32_t i = 0; i < VP; i++) {
+            const uint32_t idx = tid + 256 * i, kp = idx / (DV / 4), d = idx % (DV / 4) * 4, t = kt * KT + 2 * kp;
+            const T* src = vbuf + (size_t)(t - kv_lo) * vst + head * sh.vdim + d;
+            const bool in = d < sh.vdim;
+            x4 z;
+#pragma unroll
+            for (int e = 0; e < 4; e++) z[e] = (T)0.f;
+            va[i] = in && t < total ? *reinterpret_cast<const x4*>(src) : z;
+            vb[i] = in && t + 1 < total ? *reinterpret_cast<const x4*>(src + vst) : z;
+        }
+    };
+    auto store_tile = [&]() {
+#pragma unroll
+        for (uint32_t i = 0; i < KP; i++) {
+            const uint32_t idx = tid + 256 * i, key = idx / (DQ / 8), d = idx % (DQ / 8) * 8;
+            store8(Ks + key * KS + d, kreg[i]);
+        }
+        // the two keys' values of one column side by side
+#pragma unroll
+        for (uint32_t i = 0; i < VP; i++) {
+            const uint32_t idx = tid + 256 * i, kp = idx / (DV / 4), d = idx % (DV / 4) * 4;
+#pragma unroll
+            for (int e = 0; e < 4; e++) {
+                struct __attribute__((aligned(2 * sizeof(T)))) Pair { T a, b; } p = {va[i][e], vb[i][e]};
+                *reinterpret_cast<Pair*>(Vt + (d + e) * VS + 2 * kp) = p;
+            }
+        }
+    };
+
+    load_tile(tile0);
+    for (uint32_t kt = tile0; kt < ntiles; kt++) {
+        __syncthreads();                      // the previous tile has been read
+        store_tile();
+        __syncthreads();
+        if (kt + 1 < ntiles) load_tile(kt + 1);
+        const uint32_t k0 = kt * KT;
+        if (!(wave_active && k0 <= wave_max && k0 + KT > wave_lo)) continue;       // all in the wave's future, or before its windows
+        v16f sacc[2];
+#pragma unroll
+        for (int h = 0; h < 2; h++)
+#pragma unroll
+            for (int r = 0; r < 16; r++) sacc[h][r] = 0.f;
+#pragma unroll
+        for (uint32_t s = 0; s < NS; s++)
+#pragma unroll
+            for (int h = 0; h < 2; h++) sacc[h] = mma32(load8(Ks + (h * 32 + lq) * KS + 16 * s + 8 * lh), qf[s], sacc[h]);
+        if (k0 + KT - 1 > wave_min || (sh.window && k0 < first_visible(wave_max))) {
+#pragma unroll
+            for (int h = 0; h < 2; h++)
+#pragma unroll
+                for (int r = 0; r < 16; r++) {
+                    const uint32_t t = k0 + 32 * h + 8 * (r >> 2) + 4 * lh + (r & 3);
+                    sacc[h][r] = (t <= qpos && qpos - t < window) ? sacc[h][r] * c2 : -INFINITY;
+                }
+        } else {
+#pragma unroll
+            for (int h = 0; h < 2; h++)
+#pragma unroll
+                for (int r = 0; r < 16; r++) sacc[h][r] *= c2;
+        }
+        float m_tile = -INFINITY;
+#pragma unroll
+        for (int h = 0; h < 2; h++)
+#pragma unroll
+            for (int r = 0; r < 16; r++) m_tile = fmaxf(m_tile, sacc[h][r]);
+        const float m_new = fmaxf(m_run, lane_xor_max<32>(m_tile));
+        const float m_exp = m_new == -INFINITY ? 0.f : m_new;            // no key seen yet: every weight is 2^-inf = 0
+        if (__builtin_amdgcn_ballot_w64(m_new > m_run) != 0) {
+            const float alpha = m_run == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m_run - m_new);
+            l_run *= alpha;
+#pragma unroll
+            for (uint32_t d = 0; d < ND; d++)
+#pragma unroll
+                for (int r = 0; r < 16; r++) oacc[d][r] *= alpha;
+        }
+        m_run = m_new;
+#pragma unroll
+        for (int h = 0; h < 2; h++)
+#pragma unroll
+            for (int j = 0; j < 2; j++) {
+                x8 pb;
+#pragma unroll
+                for (int e = 0; e < 8; e++) {
+                    const float p = __builtin_amdgcn_exp2f(sacc[h][8 * j + e] - m_exp);
+                    l_run += p;
+                    pb[e] = (T)p;
+                }
+                // element e of lane half lh is key 32 h + 16 j + 8 (e / 4) + 4 lh + e % 4
+#pragma unroll
+                for (uint32_t d = 0; d < ND; d++) {
+                    const T* vr = Vt + (d * 32 + lq) * VS + h * 32 + 16 * j + 4 * lh;
+                    const x4 v0 = *reinterpret_cast<const x4*>(vr), v1 = *reinterpret_cast<const x4*>(vr + 8);
+                    oacc[d] = mma32((x8){v0[0], v0[1], v0[2], v0[3], v1[0], v1[1], v1[2], v1[3]}, pb, oacc[d]);
+                }
+            }
+    }
+    const float l_tot = lane_xor_add<32>(l_run);
+    if (qrow >= M) return;
+    const float inv = 1.0f / l_tot;
+#pragma unroll
+    for (uint32_t d = 0; d < ND; d++)
+#pragma unroll
+        for (int g = 0; g < 4; g++) {
+            const uint32_t c = 32 * d + 8 * g + 4 * lh;
+            if (c >= sh.vdim) continue;
+            const size_t at = (size_t)qrow * ld_out + head * sh.vdim + c;
+            const x4 gt = *reinterpret_cast<const x4*>(gate + at);
+            store4<T>(out + at, oacc[d][4 * g] * inv * (float)gt[0], oacc[d][4 * g + 1] * inv * (float)gt[1], oacc[d][4 * g + 2] * inv * (float)gt[2],
+                      oacc[d][4 * g + 3] * inv * (float)gt[3]);
+        }
+}
+
+// ---- decode ----------------------------------------------------------------------------------------------------------------
+// [RMS norm of the query latent | W_uq | rotation]; the last workgroup writes the position's cache row instead.
+template <typename T, int KS>
+__global__ __launch_bounds__(GEMV_THREADS) void latent_query_kernel(LatentShape sh, const float* __restrict__ raw, const float* __restrict__ q_norm,
+                                                                    const float* __restrict__ kv_norm, const T* __restrict__ uq, DenseEpiArgs e,
+                                                                    T* __restrict__ cache) {
+    extern __shared__ __attribute__((aligned(16))) float lq_lds[];
+    const uint32_t tid = threadIdx.x, K = sh.q_rank;
+    float* xs = lq_lds;
+    float* red = lq_lds + K;
+    if (blockIdx.x == gridDim.x - 1) {
+        store_cache_row<T>(sh, raw, kv_norm, e.cos_t, e.sin_t, e.pos_dev ? *e.pos_dev : e.base_pos, cache, red, tid, GEMV_THREADS);
+        return;
+    }
+    gemv_body<T, KS, DenseEpi::Rope>(uq, sh.q_row(), K, blockIdx.x * gemv_rows<KS>(), xs, red, e, [&]() {
+        float ss = 0.f;
+        for (uint32_t i = tid; i < K; i += GEMV_THREADS) ss = fmaf(raw[i], raw[i], ss);
+        const float inv = 1.0f / sqrtf(block_sum(ss, red, tid, GEMV_THREADS) / (float)sh.q_rank_n + sh.eps);
+        for (uint32_t i = tid; i < K; i += GEMV_THREADS) xs[i] = raw[i] * inv * q_norm[i];
+    });
+}
+
+// ql[head][r] = sum_d q[head][d] W_uk[head dim + d][r].  Workgroup = (64 columns, head): a wave reads 8 rows of 64 columns at a time.
+template <typename T>
+__global__ __launch_bounds__(256) void latent_absorb_kernel(LatentShape sh, const T* __restrict__ q, const T* __restrict__ uk, T* __restrict__ ql) {
+    __shared__ float part[32][64];
+    const uint32_t tid = threadIdx.x, lane8 = tid & 7, drow = tid >> 3, head = blockIdx.y, r0 = blockIdx.x * 64;
+    const T* qh = q + head * (sh.dim + sh.rot);
+    const T* w = uk + (size_t)head * sh.dim * sh.rank + r0 + lane8 * 8;
+    float acc[8];
+#pragma unroll
+    for (int j = 0; j < 8; j++) acc[j] = 0.f;
+    for (uint32_t d = drow; d < sh.dim; d += 32) {
+        const typename Vec<T>::x8 v = load8(w + (size_t)d * sh.rank);
+        const float x = (float)qh[d];
+#pragma unroll
+        for (int j = 0; j < 8; j++) acc[j] = fmaf((float)v[j], x, acc[j]);
+    }
+#pragma unroll
+    for (int j = 0; j < 8; j++) part[drow][lane8 * 8 + j] = acc[j];
+    __syncthreads();
+    if (tid < 64) {
+        float s = 0.f;
+#pragma unroll
+        for (int i = 0; i < 32; i++) s += part[i][tid];
+        ql[(size_t)head * sh.rank + r0 + tid] = (T)s;
+    }
+}
+
+// Attention of one row over the cached latents, 16 heads per workgroup: part blockIdx.x of the visible keys, heads 16 blockIdx.y...
+// A tile is 16 NW keys; wave w computes the scores of 16 of them (straight from the cache rows in registers, which it also lays
+// down transposed in LDS), and then the weighted latents of its share of the rank.  parts[part][head][rank + 2]: sums, maximum
+// (base 2), weight sum.
+template <typename T, int NW, int MAXT>
+__global__ __launch_bounds__(NW * 64) void latent_attn_decode_kernel(LatentShape sh, const T* __restrict__ q, const T* __restrict__ ql, const T* __restrict__ cache,
+                                                                     float* __restrict__ parts, uint32_t base_pos, const uint32_t* __restrict__ pos_dev) {
+    typedef typename Vec<T>::x8 x8;
+    constexpr uint32_t KT = 16 * NW, PAD = 16 / sizeof(T), VS = KT + PAD;
+    constexpr uint32_t KSTEPS = KT / 32;
+    static_assert(KT % 32 == 0, "the second product works 32 keys at a time");
+    extern __shared__ __attribute__((aligned(16))) uint8_t ld_lds[];
+    T* Ct = reinterpret_cast<T*>(ld_lds);                   // [rank][VS]
+    T* P = Ct + sh.rank * VS;                               // [16][VS]
+    float* smax = reinterpret_cast<float*>(P + 16 * VS);    // [NW][16]
+    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, lg = lane >> 4;
+    const uint32_t pos = pos_dev ? *pos_dev : base_pos;
+    const uint32_t lo = sh.window && pos >= sh.window ? pos - sh.window + 1 : 0;
+    const uint32_t nk = pos + 1 - lo, ntiles = (nk + KT - 1) / KT, per = (ntiles + gridDim.x - 1) / gridDim.x;
+    const uint32_t t0 = blockIdx.x * per, t1 = min(t0 + per, ntiles);
+    const uint32_t head = blockIdx.y * 16 + l16, hq = min(head, sh.heads - 1);
+    const uint32_t NS = sh.cache_row() / 32, NSR = sh.rank / 32;
+    const T* qn = ql + (size_t)hq * sh.rank + 8 * lg;
+    const T* qr = q + (size_t)hq * (sh.dim + sh.rot) + sh.dim + 8 * lg;
+    const float c2 = sh.scale * LOG2E;
+    const uint32_t rtiles = sh.rank / 16;
+
+    v4f o[MAXT];
+#pragma unroll
+    for (int i = 0; i < MAXT; i++) o[i] = (v4f){0.f, 0.f, 0.f, 0.f};
+    float m_run = -INFINITY, l_run = 0.f;
+
+    for (uint32_t tile = t0; tile < t1; tile++) {
+        const uint32_t tk = lo + tile * KT + wave * 16;          // the wave's first key
+        const T* row = cache + (size_t)min(tk + l16, pos) * sh.cache_row() + 8 * lg;
+        v4f sacc = (v4f){0.f, 0.f, 0.f, 0.f};
+        auto lay_down = [&](uint32_t s, const x8& f) {
+            // Ct[32 s + 8 lg + e][16 wave + l16]
+            if constexpr (sizeof(T) == 2) {
+                // pairs of keys: the even lane writes elements 0..3 of both keys, the odd lane 4..7
+                const uint4 b = __builtin_bit_cast(uint4, f);
+                const bool odd = l16 & 1;
+                const uint32_t give0 = odd ? b.x : b.z, give1 = odd ? b.y : b.w;
+                const uint32_t got0 = lane_xor<1>(give0), got1 = lane_xor<1>(give1);
+                const uint32_t mine0 = odd ? b.z : b.x, mine1 = odd ? b.w : b.y;
+                const uint32_t e0 = odd ? got0 : mine0, e1 = odd ? got1 : mine1;      // even key
+                const uint32_t d0 = odd ? mine0 : got0, d1 = odd ? mine1 : got1;      // odd key
+                uint32_t* dst = reinterpret_cast<uint32_t*>(Ct + (32 * s + 8 * lg + (odd ? 4 : 0)) * VS + 16 * wave + (l16 & ~1u));
+                dst[0 * (VS / 2)] = __builtin_amdgcn_perm(d0, e0, 0x05040100u);
+                dst[1 * (VS / 2)] = __builtin_amdgcn_perm(d0, e0, 0x07060302u);
+                dst[2 * (VS / 2)] = __builtin_amdgcn_perm(d1, e1, 0x05040100u);
+                dst[3 * (VS / 2)] = __builtin_amdgcn_perm(d1, e1, 0x07060302u);
+            } else {
+#pragma unroll
+                for (int e = 0; e < 8; e++) Ct[(32 * s + 8 * lg + e) * VS + 16 * wave + l16] = f[e];
+            }
+        };
+        constexpr uint32_t U = sizeof(T) == 2 ? 4 : 2;
+        uint32_t s = 0;
+        for (; s + U <= NSR; s += U) {
+            x8 f[U], g[U];
+#pragma unroll
+            for (uint32_t u = 0; u < U; u++) { f[u] = load8(row + 32 * (s + u)); g[u] = load8(qn + 32 * (s + u)); }
+#pragma unroll
+            for (uint32_t u = 0; u < U; u++) { sacc = mma16(f[u], g[u], sacc); lay_down(s + u, f[u]); }
+        }
+        for (; s < NSR; s++) {
+            const x8 f = load8(row + 32 * s);
+            sacc = mma16(f, load8(qn + 32 * s), sacc);
+            lay_down(s, f);
+        }
+        for (; s < NS; s++) sacc = mma16(load8(row + 32 * s), load8(qr + 32 * (s - NSR)), sacc);
+        // register r: key tk + 4 lg + r, this lane's head
+        float mx = -INFINITY;
+#pragma unroll
+        for (int r = 0; r < 4; r++) {
+            sacc[r] = tk + 4 * lg + r <= pos ? sacc[r] * c2 : -INFINITY;
+            mx = fmaxf(mx, sacc[r]);
+        }
+        mx = lane_xor_max<32>(lane_xor_max<16>(mx));
+        if (lane < 16) smax[wave * 16 + l16] = mx;
+        __syncthreads();
+        float m_new = m_run;
+#pragma unroll
+        for (int w = 0; w < NW; w++) m_new = fmaxf(m_new, smax[w * 16 + l16]);
+        // finite: the tile's first key is visible
+        const float alpha = m_run == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m_run - m_new);
+        m_run = m_new;
+        float p[4];
+        l_run *= alpha;
+#pragma unroll
+        for (int r = 0; r < 4; r++) { p[r] = __builtin_amdgcn_exp2f(sacc[r] - m_new); l_run += p[r]; }
+        store4<T>(P + l16 * VS + 16 * wave + 4 * lg, p[0], p[1], p[2], p[3]);
+        __syncthreads();
+#pragma unroll
+        for (int i = 0; i < MAXT; i++) {
+            const uint32_t rt = wave + i * NW;
+            if (rt < rtiles) {
+                o[i] *= alpha;
+#pragma unroll
+                for (uint32_t k = 0; k < KSTEPS; k++)
+                    o[i] = mma16(load8(Ct + (rt * 16 + l16) * VS + 32 * k + 8 * lg), load8(P + l16 * VS + 32 * k + 8 * lg), o[i]);
+            }
+        }
+        __syncthreads();
+    }
+    float* rec = parts + ((size_t)blockIdx.x * sh.heads + hq) * (sh.rank + 4);
+    l_run = lane_xor_add<32>(lane_xor_add<16>(l_run));
+    if (lane < 16) smax[wave * 16 + l16] = l_run;
+    __syncthreads();
+    if (head < sh.heads) {
+        if (t0 < t1) {
+#pragma unroll
+            for (int i = 0; i < MAXT; i++) {
+                const uint32_t rt = wave + i * NW;
+                if (rt < rtiles) *reinterpret_cast<v4f*>(rec + rt * 16 + 4 * lg) = o[i];
+            }
+        }
+        if (tid < 16) {
+            float l = 0.f;
+            for (int w = 0; w < NW; w++) l += smax[w * 16 + l16];
+            rec[sh.rank] = m_run;                  // -inf: an empty part, whose sums are not read
+            rec[sh.rank + 1] = l;
+        }
+    }
+}
+
+// [merge of the parts | W_uv | gate]: a workgroup's rows belong to one head.
+template <typename T, int KS>
+__global__ __launch_bounds__(GEMV_THREADS) void latent_value_kernel(LatentShape sh, const float* __restrict__ parts, uint32_t nparts, const T* __restrict__ uv, DenseEpiArgs e) {
+    extern __shared__ __attribute__((aligned(16))) float lv_lds[];
+    const uint32_t tid = threadIdx.x, K = sh.rank, row0 = blockIdx.x * gemv_rows<KS>();
+    const uint32_t head = row0 / sh.vdim;
+    float* xs = lv_lds;
+    float* red = lv_lds + K;
+    float* wt = red + 16;           // [SPLITS_MAX]
+    gemv_body<T, KS, DenseEpi::GateMul>(uv, sh.heads * sh.vdim, K, row0, xs, red, e, [&]() {
+        const size_t step = (size_t)sh.heads * (sh.rank + 4);
+        const float* rec = parts + (size_t)head * (sh.rank + 4);
+        if (tid < 64) {
+            const float m = tid < nparts ? rec[tid * step + sh.rank] : -INFINITY;
+            const float mx = wave_max(m);
+            const float w = m == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m - mx);
+            const float l = wave_sum(w > 0.f ? w * rec[tid * step + sh.rank + 1] : 0.f);
+            if (tid < SPLITS_MAX) wt[tid] = w / l;
+        }
+        __syncthreads();
+        for (uint32_t i = tid; i < K; i += GEMV_THREADS) {
+            float v = 0.f;
+            for (uint32_t p = 0; p < nparts; p++)
+                if (wt[p] > 0.f) v = fmaf(wt[p], rec[p * step + i], v);
+            xs[i] = v;
+        }
+    });
+}
+
+namespace {
+
+template <typename T, int DQ, int DV>
+void go_prefill(const LatentShape& sh, const void* q, const void* kbuf, const void* vbuf, const void* cache, uint32_t kv_lo, const void* gate,
+                void* out, uint32_t ld_out, uint32_t M, uint32_t base_pos, hipStream_t s) {
+    constexpr uint32_t lds = (64 * (DQ + 16 / sizeof(T)) + DV * (64 + 8 / sizeof(T))) * sizeof(T);
+    static_assert(lds <= 160 * 1024, "LDS of a compute unit");
+    static const hipError_t ok = hipFuncSetAttribute((const void*)latent_attn_prefill_kernel<T, DQ, DV>, hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+    (void)ok;
+    fh::launch(latent_attn_prefill_kernel<T, DQ, DV>, dim3((M + 127) / 128 * sh.heads), 256, lds, s, sh, (const T*)q, (const T*)kbuf, (const T*)vbuf,
+               (const T*)cache, kv_lo, (const T*)gate, (T*)out, ld_out, M, base_pos);
+}
+
+template <typename T>
+void prefill_by_size(const LatentShape& sh, const void* q, const void* kbuf, const void* vbuf, const void* cache, uint32_t kv_lo, const void* gate,
+                     void* out, uint32_t ld_out, uint32_t M, uint32_t base_pos, hipStream_t s) {
+    const uint32_t dq = sh.dim + sh.rot, dv = sh.vdim;
+#define FH_LP(DQ_, DV_) if (dq <= DQ_ && dv <= DV_) { go_prefill<T, DQ_, DV_>(sh, q, kbuf, vbuf, cache, kv_lo, gate, out, ld_out, M, base_pos, s); return; }
+    FH_LP(64, 32)
+    FH_LP(96, 64)
+    FH_LP(128, 128)
+    FH_LP(192, 128)
+    FH_LP(256, 256)
+#undef FH_LP
+}
+
+template <typename T, int NW, int MAXT>
+void go_decode(const LatentShape& sh, const LatentDecodeIo& io, hipStream_t s) {
+    constexpr uint32_t VS = 16 * NW + 16 / sizeof(T);
+    static const hipError_t ok = hipFuncSetAttribute((const void*)latent_attn_decode_kernel<T, NW, MAXT>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+    (void)ok;
+    const uint32_t lds = (sh.rank + 16) * VS * sizeof(T) + NW * 16 * 4;
+    fh::launch(latent_attn_decode_kernel<T, NW, MAXT>, dim3(latent_splits(sh, io.max_seq), (sh.heads + 15) / 16), NW * 64, lds, s, sh, (const T*)io.q,
+               (const T*)io.ql, (const T*)io.cache, io.parts, io.base_pos, io.pos_dev);
+}
+
+template <typename T, int KS>
+void go_query(const LatentShape& sh, const LatentDecodeIo& io, const DenseEpiArgs& e, hipStream_t s) {
+    static const hipError_t ok = hipFuncSetAttribute((const void*)latent_query_kernel<T, KS>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+    (void)ok;
+    fh::launch(latent_query_kernel<T, KS>, dim3((sh.q_row() + gemv_rows<KS>() - 1) / gemv_rows<KS>() + 1), GEMV_THREADS, (sh.q_rank + 16) * 4, s, sh, io.raw,
+               io.q_norm, io.kv_norm, (const T*)io.uq.p, e, (T*)io.cache);
+}
+
+template <typename T>
+void query(const LatentShape& sh, const LatentDecodeIo& io, hipStream_t s) {
+    DenseEpiArgs e;
+    e.out = io.q;
+    e.ld_out = sh.q_row();
+    e.cos_t = io.cos_t;
+    e.sin_t = io.sin_t;
+    e.base_pos = io.base_pos;
+    e.pos_dev = io.pos_dev;
+    e.head_stride = sh.dim + sh.rot;
+    e.rot_off = sh.dim;
+    e.rot_pairs = sh.rot_pairs;
+    switch (gemv_depth_split(sh.q_row(), sh.q_rank)) {
+        case 1: go_query<T, 1>(sh, io, e, s); break;
+        case 2: go_query<T, 2>(sh, io, e, s); break;
+        default: go_query<T, 4>(sh, io, e, s); break;
+    }
+}
+
+template <typename T>
+void decode(const LatentShape& sh, const LatentDecodeIo& io, hipStream_t s) {
+    fh::launch(latent_absorb_kernel<T>, dim3(sh.rank / 64, sh.heads), 256, 0, s, sh, (const T*)io.q, (const T*)io.ukv.p, (T*)io.ql);
+    if constexpr (sizeof(T) == 2) {
+        if (sh.rank <= 128) go_decode<T, 4, 2>(sh, io, s);
+        else if (sh.rank <= 512) go_decode<T, 4, 8>(sh, io, s);
+        else go_decode<T, 4, 16>(sh, io, s);
+    } else {
+        if (sh.rank <= 128) go_decode<T, 4, 2>(sh, io, s);
+        else if (sh.rank <= 512) go_decode<T, 4, 8>(sh, io, s);
+        else go_decode<T, 2, 32>(sh, io, s);
+    }
+    DenseEpiArgs e;
+    e.out = io.out;
+    e.gate = io.gate;
+    // rows of a workgroup (16 or 4) lie in one head: vdim is a multiple of 32
+    const T* uv = (const T*)io.ukv.p + (size_t)sh.heads * sh.dim * sh.rank;
+    const uint32_t N = sh.heads * sh.vdim, lds = (sh.rank + 16 + SPLITS_MAX) * 4, np = latent_splits(sh, io.max_seq);
+    if (gemv_depth_split(N, sh.rank) == 1) fh::launch(latent_value_kernel<T, 1>, dim3(N / gemv_rows<1>()), GEMV_THREADS, lds, s, sh, io.parts, np, uv, e);
+    else fh::launch(latent_value_kernel<T, 4>, dim3(N / gemv_rows<4>()), GEMV_THREADS, lds, s, sh, io.parts, np, uv, e);
+}
+
+}  // namespace
+
+bool latent_shape_supported(DType, const LatentShape& sh) {
+    return sh.dim + sh.rot <= HEAD_DIM_MAX && sh.vdim <= HEAD_DIM_MAX && sh.rank <= RANK_MAX && sh.q_rank <= dense_k_max();
+}
+
+uint32_t latent_splits(const LatentShape& sh, uint32_t max_seq) {
+    const uint32_t keys = sh.window && sh.window < max_seq ? sh.window : max_seq;
+    return std::max(1u, std::min(SPLITS_MAX, (keys + 63) / 64));
+}
+
+size_t latent_parts_bytes(const LatentShape& sh, uint32_t max_seq) {
+    return (size_t)latent_splits(sh, max_seq) * sh.heads * (sh.rank + 4) * 4;
+}
+
+void launch_latent_norm_store(DType t, const LatentShape& sh, const float* raw, const float* q_norm, const float* kv_norm, const float* cos_t,
+                              const float* sin_t, uint32_t M, uint32_t base_pos, void* cq, void* cache, hipStream_t s) {
+    if (t == DType::BF16)
+        fh::launch(latent_norm_store_kernel<__bf16>, dim3(M), 256, 0, s, sh, raw, q_norm, kv_norm, cos_t, sin_t, base_pos, (__bf16*)cq, (__bf16*)cache);
+    else
+        fh::launch(latent_norm_store_kernel<float>, dim3(M), 256, 0, s, sh, raw, q_norm, kv_norm, cos_t, sin_t, base_pos, (float*)cq, (float*)cache);
+}
+
+void launch_latent_attn_prefill(DType t, const LatentShape& sh, const void* q, const void* kbuf, const void* vbuf, const void* cache, uint32_t kv_lo,
+                                const void* gate, void* out, uint32_t ld_out, uint32_t M, uint32_t base_pos, hipStream_t s) {
+    if (t == DType::BF16) prefill_by_size<__bf16>(sh, q, kbuf, vbuf, cache, kv_lo, gate, out, ld_out, M, base_pos, s);
+    else prefill_by_size<float>(sh, q, kbuf, vbuf, cache, kv_lo, gate, out, ld_out, M, base_pos, s);
+}
+
+void launch_latent_query(DType t, const LatentShape& sh, const LatentDecodeIo& io, hipStream_t s) {
+    if (t == DType::BF16) query<__bf16>(sh, io, s);
+    else query<float>(sh, io, s);
+}
+
+void launch_latent_attn_decode(DType t, const LatentShape& sh, const LatentDecodeIo& io, hipStream_t s) {
+    if (t == DType::BF16) decode<__bf16>(sh, io, s);
+    else decode<float>(sh, io, s);
+}
+
+}  // namespace fh

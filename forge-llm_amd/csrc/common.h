@@ -252,6 +252,99 @@ void launch_attn_exact(bool batch_order, const float* q, uint32_t q_stride, cons
 size_t attn_exact_decode_workspace_bytes(uint32_t heads, uint32_t hd, uint32_t max_rows);
 uint32_t attn_exact_max_window();
 
+// dense.hip — matrices in bfloat16 or 32-bit, row-major [N][K], K a multiple of 64 (zero padded), N a multiple of 4 except
+// for DenseEpi::F32.  Activations are rows of the same type, 16-byte aligned, lda a multiple of 8.
+enum class DType : uint32_t { F32 = 0, BF16 = 30 };       // GGML type ids
+inline size_t dtype_size(DType t) { return t == DType::F32 ? 4 : 2; }
+struct DenseWeight {
+    void* p = nullptr;
+    uint32_t N = 0, K = 0;
+};
+// An elementwise norm, tanh(alpha * x) * w + b; w == nullptr: the identity.
+struct DynTanh {
+    const float* w = nullptr;
+    const float* b = nullptr;
+    float alpha = 0.f;
+};
+enum class DenseEpi {
+    F32,        // f32[m][n] = v
+    RawGate,    // columns below `split`: f32[m][n] = v; the others: out[m][n - split] = sigmoid(v)
+    Rope,       // heads of head_stride columns: the pairs (rot_off + 2 i, rot_off + 2 i + 1), i < rot_pairs, turn by the angle of (position, i); out = the result
+    Split,      // columns below `split` go to out, the others to out2
+    GateMul,    // out = v * gate
+    SiluPair,   // columns 2 i and 2 i + 1 are gate and up: out[m][i] = silu(gate) * up
+    Residual,   // a = post(v) (+ f32 if add); f32 = a; out = next(a)
+};
+struct DenseEpiArgs {
+    float* f32 = nullptr;
+    uint32_t ld_f32 = 0;
+    void* out = nullptr;
+    uint32_t ld_out = 0;
+    void* out2 = nullptr;
+    uint32_t ld_out2 = 0;
+    uint32_t split = 0;
+    const void* gate = nullptr;      // [m][ld_out]
+    DynTanh post, next;
+    int add = 0;
+    const float* cos_t = nullptr;    // [position][rot_pairs]
+    const float* sin_t = nullptr;
+    uint32_t base_pos = 0;
+    const uint32_t* pos_dev = nullptr;
+    uint32_t head_stride = 1, rot_off = 0, rot_pairs = 0;
+};
+// y = a W^T over M rows, then the epilogue.  One row runs as a matrix-vector kernel.
+void launch_dense(DType t, const DenseWeight& w, const void* a, uint32_t lda, uint32_t M, DenseEpi mode, const DenseEpiArgs& e, hipStream_t s);
+uint32_t dense_k_max();
+// x[m] = table[token[m]] * scale (f32, rows of ldx, zero past `width`), out = next(x), out2 (optional) = x; counts as in launch_embedding.
+void launch_dense_embedding(DType t, const void* table, uint32_t width, float scale, const uint32_t* tokens_dev, uint32_t M, float* x,
+                            uint32_t ldx, const DynTanh& next, void* out, uint32_t ld_out, void* out2, uint32_t ld_out2, uint32_t* counts, hipStream_t s);
+// out[i] = a[rows[i]] for n rows of `width` elements
+void launch_gather_rows(DType t, const void* a, uint32_t lda, const uint32_t* rows_dev, uint32_t n, uint32_t width, void* out, uint32_t ld_out, hipStream_t s);
+
+// attn_latent.hip — attention whose keys and values are linear maps of one cached latent vector per position, beside one rotated
+// key part that all heads share.  Sizes are the padded ones of the buffers (multiples of 32; the latent a multiple of 64).
+struct LatentShape {
+    uint32_t heads = 0, dim = 0, rot = 0, vdim = 0, rank = 0, q_rank = 0;
+    uint32_t rank_n = 0, q_rank_n = 0;       // elements the two RMS norms count
+    uint32_t rot_pairs = 0;
+    uint32_t window = 0;                     // 0: every earlier position
+    float scale = 0.f, eps = 0.f;
+    __host__ __device__ uint32_t cache_row() const { return rank + rot; }
+    __host__ __device__ uint32_t raw_row() const { return q_rank + rank + rot; }
+    __host__ __device__ uint32_t q_row() const { return heads * (dim + rot); }
+};
+bool latent_shape_supported(DType t, const LatentShape& sh);
+// raw f32 [M][q_rank | rank | rot] -> cq [M][q_rank] = RMSnorm * q_norm; cache row of the position = RMSnorm * kv_norm | rotated part
+void launch_latent_norm_store(DType t, const LatentShape& sh, const float* raw, const float* q_norm, const float* kv_norm, const float* cos_t,
+                              const float* sin_t, uint32_t M, uint32_t base_pos, void* cq, void* cache, hipStream_t s);
+// Prompt form: keys and values expanded per head, kbuf [positions kv_lo..][heads][dim], vbuf [..][heads][vdim] (kv_lo a multiple of
+// 64), the rotated key part from the cache; out [M][ld_out] = attention * gate.
+void launch_latent_attn_prefill(DType t, const LatentShape& sh, const void* q, const void* kbuf, const void* vbuf, const void* cache, uint32_t kv_lo,
+                                const void* gate, void* out, uint32_t ld_out, uint32_t M, uint32_t base_pos, hipStream_t s);
+// One row at pos_dev ? *pos_dev : base_pos, four launches: [norm of the query latent | W_uq | rotation] beside the new cache row,
+// queries taken to the latent space (W_uk^T q per head), attention over the cached latents in up to latent_splits() parts, and
+// [merge of the parts | W_uv | gate].
+struct LatentDecodeIo {
+    const float* raw;                  // [raw_row()]
+    const float* q_norm;
+    const float* kv_norm;
+    const float* cos_t;
+    const float* sin_t;
+    DenseWeight uq, ukv;               // ukv: [heads * dim rows of W_uk | heads * vdim rows of W_uv][rank]
+    void* q;                           // [q_row()]
+    void* ql;                          // [heads][rank]
+    void* cache;
+    float* parts;                      // latent_parts_bytes()
+    const void* gate;
+    void* out;
+    uint32_t max_seq, base_pos;
+    const uint32_t* pos_dev;
+};
+uint32_t latent_splits(const LatentShape& sh, uint32_t max_seq);
+size_t latent_parts_bytes(const LatentShape& sh, uint32_t max_seq);
+void launch_latent_query(DType t, const LatentShape& sh, const LatentDecodeIo& io, hipStream_t s);
+void launch_latent_attn_decode(DType t, const LatentShape& sh, const LatentDecodeIo& io, hipStream_t s);
+
 // decode_persistent.hip — the whole decode step as one resident kernel (fast mode only)
 struct PdLayerIn {
     const QWeight* qkv;        // uniform models: the fused matrices

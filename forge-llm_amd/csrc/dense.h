@@ -1,0 +1,129 @@
+// Dense (bfloat16 or 32-bit) matrices: element types, matrix-unit fragments and the epilogues that the matrix-matrix and the
+// matrix-vector kernels share.  T is the storage type of weights and activations: __bf16 or float.  Sums are 32-bit in both.
+#pragma once
+
+#include <hip/hip_runtime.h>
+#include <math.h>
+#include <stdint.h>
+
+#include "common.h"
+#include "device_utils.h"
+
+namespace fh {
+
+typedef float v4f __attribute__((ext_vector_type(4)));
+typedef float v8f __attribute__((ext_vector_type(8)));
+typedef float v16f __attribute__((ext_vector_type(16)));
+typedef __bf16 v4bf __attribute__((ext_vector_type(4)));
+typedef __bf16 v8bf __attribute__((ext_vector_type(8)));
+
+// Four and eight elements of a row in registers.
+template <typename T> struct Vec;
+template <> struct Vec<__bf16> { typedef v4bf x4; typedef v8bf x8; };
+template <> struct Vec<float> { typedef v4f x4; typedef v8f x8; };
+
+template <typename T> __device__ __forceinline__ typename Vec<T>::x8 load8(const T* p) {
+    if constexpr (sizeof(T) == 2) return *reinterpret_cast<const v8bf*>(p);
+    else {
+        const v4f a = reinterpret_cast<const v4f*>(p)[0], b = reinterpret_cast<const v4f*>(p)[1];
+        return (v8f){a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
+    }
+}
+template <typename T> __device__ __forceinline__ void store8(T* p, typename Vec<T>::x8 v) {
+    if constexpr (sizeof(T) == 2) *reinterpret_cast<v8bf*>(p) = v;
+    else {
+        reinterpret_cast<v4f*>(p)[0] = (v4f){v[0], v[1], v[2], v[3]};
+        reinterpret_cast<v4f*>(p)[1] = (v4f){v[4], v[5], v[6], v[7]};
+    }
+}
+template <typename T> __device__ __forceinline__ typename Vec<T>::x8 zero8() {
+    typename Vec<T>::x8 z;
+#pragma unroll
+    for (int e = 0; e < 8; e++) z[e] = (T)0.0f;
+    return z;
+}
+template <typename T> __device__ __forceinline__ void store4(T* p, float a, float b, float c, float d) {
+    typename Vec<T>::x4 v;
+    v[0] = (T)a; v[1] = (T)b; v[2] = (T)c; v[3] = (T)d;
+    *reinterpret_cast<typename Vec<T>::x4*>(p) = v;
+}
+
+// D += A B on the matrix unit with both operands as "8 elements per lane" fragments.  32x32 tile, depth 16: lane l holds row
+// (column) l % 32 and the depths 8 (l / 32) + 0..7; the result lane l holds column l % 32 and, in register r, row
+// 8 (r / 4) + 4 (l / 32) + r % 4.  The 32-bit form is eight depth-2 instructions over the same fragments (element e of the two
+// lane halves forms one of them): full single precision.
+__device__ __forceinline__ v16f mma32(v8bf a, v8bf b, v16f c) { return __builtin_amdgcn_mfma_f32_32x32x16_bf16(a, b, c, 0, 0, 0); }
+__device__ __forceinline__ v16f mma32(v8f a, v8f b, v16f c) {
+#pragma unroll
+    for (int e = 0; e < 8; e++) c = __builtin_amdgcn_mfma_f32_32x32x2f32(a[e], b[e], c, 0, 0, 0);
+    return c;
+}
+// 16x16 tile, depth 32: lane l holds row (column) l % 16 and the depths 8 (l / 16) + 0..7; the result lane l holds column l % 16
+// and, in register r, row 4 (l / 16) + r.
+__device__ __forceinline__ v4f mma16(v8bf a, v8bf b, v4f c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
+__device__ __forceinline__ v4f mma16(v8f a, v8f b, v4f c) {
+#pragma unroll
+    for (int e = 0; e < 8; e++) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a[e], b[e], c, 0, 0, 0);
+    return c;
+}
+
+// Dynamic Tanh, an elementwise norm: tanh(alpha * x) * w + b.  w == nullptr: x itself.
+__device__ __forceinline__ float dyn_tanh(const DynTanh& t, uint32_t n, float x) { return t.w ? tanhf(t.alpha * x) * t.w[n] + t.b[n] : x; }
+__device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float silu_f(float z) { return z / (1.0f + expf(-z)); }
+
+// What happens to the results (m, n .. n + 3) of a product; n is a multiple of 4.
+template <typename T, DenseEpi MODE>
+__device__ __forceinline__ void dense_epilogue(const DenseEpiArgs& e, uint32_t m, uint32_t n, uint32_t N, const float* v) {
+    if constexpr (MODE == DenseEpi::F32) {
+        float* y = e.f32 + (size_t)m * e.ld_f32 + n;
+#pragma unroll
+        for (int i = 0; i < 4; i++)
+            if (n + i < N) y[i] = v[i];
+    } else if constexpr (MODE == DenseEpi::RawGate) {
+        if (n < e.split) *reinterpret_cast<float4*>(e.f32 + (size_t)m * e.ld_f32 + n) = make_float4(v[0], v[1], v[2], v[3]);
+        else store4<T>((T*)e.out + (size_t)m * e.ld_out + (n - e.split), sigmoid_f(v[0]), sigmoid_f(v[1]), sigmoid_f(v[2]), sigmoid_f(v[3]));
+    } else if constexpr (MODE == DenseEpi::Rope) {
+        const uint32_t j = n % e.head_stride;
+        float a[4] = {v[0], v[1], v[2], v[3]};
+        if (j >= e.rot_off && (j - e.rot_off) / 2 < e.rot_pairs) {
+            const uint32_t p = (e.pos_dev ? *e.pos_dev : e.base_pos) + m, i = (j - e.rot_off) / 2;
+            const float* ct = e.cos_t + (size_t)p * e.rot_pairs;
+            const float* st = e.sin_t + (size_t)p * e.rot_pairs;
+            const float c0 = ct[i], s0 = st[i];
+            a[0] = v[0] * c0 - v[1] * s0;
+            a[1] = v[1] * c0 + v[0] * s0;
+            if (i + 1 < e.rot_pairs) {
+                const float c1 = ct[i + 1], s1 = st[i + 1];
+                a[2] = v[2] * c1 - v[3] * s1;
+                a[3] = v[3] * c1 + v[2] * s1;
+            }
+        }
+        store4<T>((T*)e.out + (size_t)m * e.ld_out + n, a[0], a[1], a[2], a[3]);
+    } else if constexpr (MODE == DenseEpi::Split) {
+        T* y = n < e.split ? (T*)e.out + (size_t)m * e.ld_out + n : (T*)e.out2 + (size_t)m * e.ld_out2 + (n - e.split);
+        store4<T>(y, v[0], v[1], v[2], v[3]);
+    } else if constexpr (MODE == DenseEpi::GateMul) {
+        const T* g = (const T*)e.gate + (size_t)m * e.ld_out + n;
+        store4<T>((T*)e.out + (size_t)m * e.ld_out + n, v[0] * (float)g[0], v[1] * (float)g[1], v[2] * (float)g[2], v[3] * (float)g[3]);
+    } else if constexpr (MODE == DenseEpi::SiluPair) {
+        T* y = (T*)e.out + (size_t)m * e.ld_out + n / 2;
+        y[0] = (T)(silu_f(v[0]) * v[1]);
+        y[1] = (T)(silu_f(v[2]) * v[3]);
+    } else if constexpr (MODE == DenseEpi::Residual) {
+        float4* xp = reinterpret_cast<float4*>(e.f32 + (size_t)m * e.ld_f32 + n);
+        float a[4];
+#pragma unroll
+        for (int i = 0; i < 4; i++) a[i] = dyn_tanh(e.post, n + i, v[i]);
+        if (e.add) {
+            const float4 x = *xp;
+            a[0] += x.x; a[1] += x.y; a[2] += x.z; a[3] += x.w;
+        }
+        *xp = make_float4(a[0], a[1], a[2], a[3]);
+#pragma unroll
+        for (int i = 0; i < 4; i++) a[i] = dyn_tanh(e.next, n + i, a[i]);
+        store4<T>((T*)e.out + (size_t)m * e.ld_out + n, a[0], a[1], a[2], a[3]);
+    }
+}
+
+}  // namespace fh

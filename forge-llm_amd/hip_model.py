@@ -8,6 +8,7 @@ Same surface as `MetalModel` in the reference (crates/forgellm-codegen-metal/src
 ForgeHipError here.
 """
 import ctypes as C
+import os
 
 import numpy as np
 
@@ -60,6 +61,28 @@ class HipModel:
         self.vocab = int(cfg["vocab"])
         return self
 
+    @classmethod
+    def from_folder(cls, path: str, max_seq: int = 0, dtype: str = "bfloat16"):
+        """Model from a folder with config.json and model.safetensors; config.json's "architecture" picks the network from the
+        library's registry.  dtype: "bfloat16" or "float32" (everything in 32-bit).  max_seq = 0: 4096 positions."""
+        from . import BF16, F32, Config, check, lib
+        L = lib()
+        self = cls.__new__(cls)
+        self._lib, self._check, self._h = L, check, None
+        h = C.c_void_p()
+        check(L.forge_hip_model_create_from_folder(str(path).encode(), int(max_seq), {"bfloat16": BF16, "float32": F32}[dtype], 0, C.byref(h)))
+        self._h = h
+        self._cfg = Config()
+        check(L.forge_hip_model_config(h, C.byref(self._cfg)))
+        self.config = {name: getattr(self._cfg, name) for name, _ in Config._fields_}
+        self.vocab = int(self._cfg.vocab)
+        return self
+
+    @classmethod
+    def from_path(cls, path: str, max_seq: int = 0, **kw):
+        """A model from what `path` is: a folder (from_folder) or a GGUF file (from_gguf)."""
+        return (cls.from_folder if os.path.isdir(path) else cls.from_gguf)(path, max_seq, **kw)
+
     # -- MetalModel::forward / model::forward
     def forward(self, token_id: int) -> np.ndarray:
         out = np.empty(self.vocab, np.float32)
@@ -83,6 +106,22 @@ class HipModel:
         out = np.empty(self.vocab, np.float32)
         self._check(self._lib.forge_hip_prefill_batch(self._h, t.ctypes.data_as(C.c_void_p), t.size,
                                                       out.ctypes.data_as(C.c_void_p)))
+        return out
+
+    def prefill_logits(self, tokens, want) -> np.ndarray:
+        """forward_prefill with the logits of the rows `want` (indices into `tokens`): [len(want), vocab]."""
+        t = np.ascontiguousarray(tokens, dtype=np.uint32)
+        w = np.ascontiguousarray(want, dtype=np.uint64)
+        out = np.empty((w.size, self.vocab), np.float32)
+        self._check(self._lib.forge_hip_prefill_logits(self._h, t.ctypes.data_as(C.c_void_p), t.size, w.ctypes.data_as(C.c_void_p), w.size,
+                                                       out.ctypes.data_as(C.c_void_p)))
+        return out
+
+    def prefill_residuals(self, tokens) -> np.ndarray:
+        """Residual stream after every layer run for `tokens` fed to an empty cache (the model is reset): [runs, tokens, hidden]."""
+        t = np.ascontiguousarray(tokens, dtype=np.uint32)
+        out = np.empty((int(self._lib.forge_hip_model_layer_runs(self._h)), t.size, int(self.config["hidden"])), np.float32)
+        self._check(self._lib.forge_hip_prefill_residuals(self._h, t.ctypes.data_as(C.c_void_p), t.size, out.ctypes.data_as(C.c_void_p)))
         return out
 
     # -- MetalModel::forward_profile: per-stage device time of one eager decode step

@@ -84,6 +84,8 @@ extern "C" {
 #define FORGE_HIP_Q8_0 8u
 #define FORGE_HIP_Q4_K 12u /* op level only: forge_hip_qweight_create + forge_hip_gemv_q */
 #define FORGE_HIP_Q6_K 14u
+#define FORGE_HIP_F32 0u   /* dense models only: forge_hip_model_create_from_folder */
+#define FORGE_HIP_BF16 30u
 
 /* Mirrors the fields of ModelConfig (crates/forgellm-frontend/src/ir.rs:484-519) that the
  * code generators read. */
@@ -160,6 +162,12 @@ int32_t forge_hip_forward_greedy(forge_hip_model* m, uint32_t token, uint32_t* n
  * `logits_host` is non-NULL it receives the logits of the LAST token (the CPU signature);
  * NULL skips the lm_head (the Metal signature). */
 int32_t forge_hip_prefill_batch(forge_hip_model* m, const uint32_t* tokens_host, uint64_t n, float* logits_host);
+
+/* The same with the logits of any rows of the prompt: row want_host[i] of these n tokens (0-based, any order, repeats allowed)
+ * goes to logits_host[i * vocab ..].  n_want = 0: no logits.  For perplexity runs and replays of given token ids; the
+ * reference returns the last row's only. */
+int32_t forge_hip_prefill_logits(forge_hip_model* m, const uint32_t* tokens_host, uint64_t n, const uint64_t* want_host, uint64_t n_want,
+                                 float* logits_host);
 
 /* MetalModel::forward_profile (metal:5307-5330: one decode step with a wait per stage, timings
  * printed).  Here: one decode step launched eagerly with a pair of events attached to every kernel
@@ -430,6 +438,26 @@ int32_t forge_hip_quantize_kquant(uint32_t ggml_type, const float* data_host, ui
 /* open + config + export_weights + forge_hip_model_create; a file that forge_hip_gguf_config_mixed finds to hold several
  * formats (or a K-quant lm_head) goes through the _mixed functions and forge_hip_model_create_mixed instead. */
 int32_t forge_hip_model_create_from_gguf(const char* path, uint32_t max_seq, uint32_t flags, forge_hip_model** out);
+
+/* ---------------- model folders (config.json + model.safetensors) ----------------
+ * Designs that the reference does not have, described layer by layer in a config.json whose "architecture" picks an entry of the
+ * library's registry (checkpoint.cpp): "Vabirax", a decoder of latent-attention layers (queries and keys / values through
+ * low-rank latents, one rotated key part shared by all heads, a sliding window, a sigmoid gate on the heads' output) and gated
+ * feed-forwards, Dynamic Tanh ahead of and behind every sublayer, part of the layers looped with a cache per pass.  The
+ * handle is an ordinary model: forward, forward_greedy, prefill, profile, repeat penalty and reset work as documented above
+ * (forge_hip_model_set_kv_pages and forge_hip_model_read_kv: this network has a flat cache of latents, they are refused).
+ * dtype: FORGE_HIP_BF16 (weights, activations and cache in bfloat16, 32-bit sums; norms, rotation, scores, softmax and the
+ * residual stream in 32-bit) or FORGE_HIP_F32 (everything in 32-bit).  max_seq = 0: 4096 positions.  flags: 0. */
+int32_t forge_hip_model_create_from_folder(const char* dir, uint32_t max_seq, uint32_t dtype, uint32_t flags, forge_hip_model** out);
+/* The sizes config.json gives, without a GPU (per-layer sizes: the first layer's; inter: the largest; max_seq and formats: 0). */
+int32_t forge_hip_folder_config(const char* dir, forge_hip_config* out);
+/* The configuration a handle was created with (any network). */
+int32_t forge_hip_model_config(const forge_hip_model* m, forge_hip_config* out);
+/* Debug/parity: the residual stream after every layer run (a looped layer counts each time) for n tokens fed to an empty cache,
+ * [forge_hip_model_layer_runs()][n][hidden] floats; n at most one prompt chunk (4096, max_seq).  The model is reset
+ * afterwards.  Model folders only. */
+uint32_t forge_hip_model_layer_runs(const forge_hip_model* m);
+int32_t forge_hip_prefill_residuals(forge_hip_model* m, const uint32_t* tokens_host, uint64_t n, float* out_host);
 
 /* ---------------- sampling (the loop of the generated main.rs, project.rs:714-751) ----------------
  * The reference's default generation is greedy WITH a repeat penalty of 1.1 (project.rs:607-611): after every
