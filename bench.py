@@ -377,6 +377,125 @@ def ops_table(fh, reps=10):
     print(json.dumps({"ops_table": rows, "reps": reps}))
 
 
+def vabirax_costs(cfg, prompt, context, es=2):
+    """Per stage: bytes one decode step reads at `context` cached positions (weights once, cache rows of the window once), and
+    multiply-add operations of a prompt of `prompt` tokens (attention: query-key pairs inside the window)."""
+    W, dec, pre = cfg["width"], {}, {}
+
+    def add(d, k, v):
+        d[k] = d.get(k, 0) + v
+
+    loop = cfg.get("loop")
+    n = len(cfg["layers"])
+    order = list(range(n)) if not loop else (list(range(loop["start"])) + list(range(loop["start"], loop["stop"])) * loop["times"]
+                                             + list(range(loop["stop"], n)))
+    for i in order:
+        m, ff = cfg["layers"][i]["mixer"], (cfg["layers"][i]["mlp"] or {"ff": 0})["ff"]
+        H, dq = m["heads"], m["dim"] + m["rot_dim"]
+        win = m.get("mask", {}).get("size") or 1 << 30
+        latent = H * (m["dim"] + m["vdim"]) * m["kv_rank"]
+        proj = (m["q_rank"] + m["kv_rank"] + m["rot_dim"] + H * m["vdim"]) * W + H * dq * m["q_rank"]
+        if loop and i == loop["start"]:
+            proj += 2 * W * W
+        add(dec, "qkv_matmul", proj * es)
+        add(dec, "attention", latent * es + min(win, context) * (m["kv_rank"] + m["rot_dim"]) * es)
+        add(dec, "o_matmul", H * m["vdim"] * W * es)
+        add(dec, "gate_up_matmul", 2 * ff * W * es)
+        add(dec, "down_matmul", ff * W * es)
+        pairs = sum(min(win, p + 1) for p in range(prompt))
+        add(pre, "qkv_matmul", 2 * prompt * (proj + latent))
+        add(pre, "attention", 2 * pairs * H * (dq + m["vdim"]))
+        add(pre, "o_matmul", 2 * prompt * H * m["vdim"] * W)
+        add(pre, "gate_up_matmul", 4 * prompt * ff * W)
+        add(pre, "down_matmul", 2 * prompt * ff * W)
+    dec["lm_head_matmul"] = cfg["vocab"] * W * es
+    return dec, pre
+
+
+def vabirax_bench(fh, args):
+    """--vabirax: prefill and decode throughput of the Vabirax design (random bfloat16 weights) at a size that resembles a real
+    model's layers, per stage against its roofline, and the Llama-family model of the same width, depth and feed-forward beside
+    it (Q8_0; its decode step both as a kernel sequence, the like of this design's, and as the resident kernel).  One JSON line."""
+    import json as js
+    import tempfile
+    import numpy as np
+    import torch
+    cfg = getattr(fh.synth, "vabirax_" + args.vabirax)()
+    prompt = fh.synth.uniform_ids(args.seed + 1, args.prompt_tokens, cfg["vocab"])
+    max_seq = (args.prompt_tokens + 2 * (args.warmup + args.steps) + 64 + 1023) // 1024 * 1024
+
+    def measure(model):
+        model.forward_prefill_batch(prompt)
+        times = []
+        for _ in range(3):
+            model.reset()
+            torch.cuda.synchronize()
+            t0 = time.perf_counter()
+            logits = model.forward_prefill(prompt)
+            torch.cuda.synchronize()
+            times.append(time.perf_counter() - t0)
+        assert np.all(np.isfinite(logits))
+        t_decode, tok = timed_decode(model, fh.ops.argmax_host(logits), args.warmup, args.steps)
+        context = model.pos
+        prof = [model.forward_profile(tok) for _ in range(8)]
+        dec = {s: (float(np.median([p[s][0] for p in prof])) * 1e3, prof[0][s][1]) for s in prof[0]}
+        model.reset()
+        pre = model.prefill_profile(prompt)
+        return {"prefill_tok_per_s": round(len(prompt) / min(times), 1), "prefill_ms": round(min(times) * 1e3, 3),
+                "decode_tok_per_s": round(args.steps / t_decode, 1), "ms_per_step": round(t_decode / args.steps * 1e3, 4),
+                "decode_launches": model.decode_launches}, dec, pre, context
+
+    def rooflines(dec, pre, dec_bytes, pre_ops, mfma_peak):
+        return ({s: {"us": round(dec[s][0], 1), "launches": dec[s][1], "GB/s": round(dec_bytes[s] / dec[s][0] / 1e3, 1),
+                     "frac": round(dec_bytes[s] / dec[s][0] / 1e3 / 8000, 4)} for s in dec_bytes},
+                {s: {"ms": round(pre[s][0], 3), "TOP/s": round(pre_ops[s] / pre[s][0] / 1e9, 1),
+                     "frac": round(pre_ops[s] / pre[s][0] / 1e9 / mfma_peak[s], 4)} for s in pre_ops})
+
+    with tempfile.TemporaryDirectory() as tmp:
+        t0 = time.perf_counter()
+        fh.synth.write_model_folder(tmp, cfg, fh.synth.vabirax_stream(cfg, args.seed))
+        t_write = time.perf_counter() - t0
+        print("written in %.1f s" % t_write, file=sys.stderr, flush=True)
+        nbytes = os.path.getsize(os.path.join(tmp, "model.safetensors"))
+        t0 = time.perf_counter()
+        model = fh.HipModel.from_folder(tmp, max_seq)
+        t_load = time.perf_counter() - t0
+    print("loaded in %.1f s" % t_load, file=sys.stderr, flush=True)
+    line, dec, pre, context = measure(model)
+    model.close()
+    dec_bytes, pre_ops = vabirax_costs(cfg, len(prompt), context)
+    line["decode_stages"], line["prefill_stages"] = rooflines(dec, pre, dec_bytes, pre_ops, dict.fromkeys(pre_ops, 2500))
+    line["decode_other_us"] = {s: round(v[0], 1) for s, v in dec.items() if s not in dec_bytes and v[1]}
+    line["prefill_other_ms"] = {s: round(v[0], 3) for s, v in pre.items() if s not in pre_ops and v[1]}
+
+    lcfg = getattr(fh.synth, "llama32_" + args.vabirax)(fh.Q8_0, max_seq=max_seq)
+    blob = fh.synth.make_weights_blob(lcfg, seed=args.seed, threads=16)
+    print("Llama weights made", file=sys.stderr, flush=True)
+    gl = gemv_launch_bytes(fh, lcfg)
+    H = lcfg["heads"] * lcfg["head_dim"]
+    n = len(prompt)
+    _, attn = prefill_flops(lcfg, n)
+    L, W, I = lcfg["layers"], lcfg["hidden"], lcfg["inter"]
+    KV = lcfg["kv_heads"] * lcfg["head_dim"]
+    l_ops = {"qkv_matmul": 2 * n * L * W * (H + 2 * KV), "attention": attn, "o_matmul": 2 * n * L * W * H, "gate_up_matmul": 4 * n * L * W * I,
+             "down_matmul": 2 * n * L * W * I}
+    peak = {s: 2500 if s == "attention" else 5000 for s in l_ops}
+    closest = {}
+    for name, env in (("kernel_sequence", "0"), ("resident_kernel", "1")):
+        os.environ["FORGE_HIP_PERSIST"] = env
+        model = fh.HipModel(lcfg, blob)
+        closest[name], dec, pre, context = measure(model)
+        model.close()
+        gl["attention"] = L * context * 2 * KV * 2
+        closest[name]["decode_stages"], closest[name]["prefill_stages"] = rooflines(dec, pre, gl, l_ops, peak)
+    print(js.dumps({"metric": "decode tok/s (Vabirax %s shape, bfloat16, 1 GPU)" % args.vabirax, "value": line["decode_tok_per_s"], "unit": "tok/s",
+                    "n_gpus": 1, "steps": args.steps, "warmup": args.warmup, "ms_per_step": line["ms_per_step"], "higher_is_better": True,
+                    "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+                    "config": {"model": "Vabirax " + args.vabirax, "prompt_tokens": n, "weights_bytes": nbytes, "write_s": round(t_write, 1),
+                               "load_s": round(t_load, 1)},
+                    "vabirax": line, "closest_model": {"model": "Llama-3.2-%s shape, Q8_0" % args.vabirax.upper(), **closest}}))
+
+
 def main():
     global PROMPT_TOKENS
     ap = argparse.ArgumentParser()
@@ -399,6 +518,8 @@ def main():
                     help="length of the prompt (default: the 2502 tokens the metric is quoted on); the cache is sized to fit")
     ap.add_argument("--ops-table", action="store_true",
                     help="instead of the model benchmark, run the isolated kernels at the benchmark configurations' sizes")
+    ap.add_argument("--vabirax", choices=("1b", "3b"),
+                    help="instead of the default workload, the Vabirax design at this size beside the Llama-family model of the same size")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this build measures ONE GPU; --gpus must be 1 (no multi-GPU path exists to run)", file=sys.stderr)
@@ -410,6 +531,9 @@ def main():
     fh.require_gpu()
     if args.ops_table:
         ops_table(fh)
+        return
+    if args.vabirax:
+        vabirax_bench(fh, args)
         return
     wd = fh.Q8_0 if args.format == "q8_0" else fh.Q4_0
     PROMPT_TOKENS = args.prompt_tokens

@@ -245,3 +245,142 @@ def decode_weight_bytes(cfg: dict) -> int:
     wt = cfg["wdtype"]
     per_layer = mat(QKS, H, wt) + 2 * mat(KV, H, wt) + mat(H, QKS, wt) + 2 * mat(I, H, wt) + mat(H, I, wt)
     return cfg["layers"] * per_layer + mat(cfg["vocab"], H, cfg["lm_head_dtype"])
+
+
+# ---- model folders (config.json + model.safetensors) ----------------------------------------------------------------------
+
+def vabirax_layer(heads, dim, rot_dim, vdim, q_rank, kv_rank, ff, window, scale=None, base=10000.0, rot_dims=None) -> dict:
+    """One entry of a Vabirax config's layer list; ff None: no feed-forward, window None: no mask."""
+    mixer = {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "q_rank": q_rank, "kv_rank": kv_rank,
+             "scale": (dim + rot_dim) ** -0.5 if scale is None else scale, "rot": {"base": base, "dims": rot_dims or rot_dim}}
+    if window:
+        mixer["mask"] = {"size": window}
+    return {"type": "latent_attention", "mixer": mixer, "mlp": None if ff is None else {"kind": "dense", "ff": ff}}
+
+
+def vabirax_config(width, vocab, layers, loop=None, embedding_scale=1.0, eps=1e-5) -> dict:
+    """layers: vabirax_layer() entries; loop: (start, stop, times) or None."""
+    c = {"architecture": "Vabirax", "width": width, "vocab": vocab, "embedding": {"scale": embedding_scale}, "norm": {"eps": eps},
+         "layers": layers}
+    if loop:
+        c["loop"] = dict(zip(("start", "stop", "times"), loop))
+    return c
+
+
+def vabirax_shapes(config) -> dict:
+    """{tensor name: shape} of a Vabirax checkpoint."""
+    w, out = config["width"], {}
+
+    def norm(name):
+        out[name], out[name + ".b"], out[name + ".alpha"] = (w,), (w,), ()
+
+    out["embed"] = (config["vocab"], w)
+    if config.get("loop"):
+        out["loop.in"] = (w, 2 * w)
+    for i, layer in enumerate(config["layers"]):
+        m, n = layer["mixer"], "l%d." % i
+        H = m["heads"]
+        norm(n + "norm1")
+        norm(n + "norm1b")
+        for name, shape in (("dq", (m["q_rank"], w)), ("dq.norm", (m["q_rank"],)), ("uq", (H * (m["dim"] + m["rot_dim"]), m["q_rank"])),
+                            ("dkv", (m["kv_rank"] + m["rot_dim"], w)), ("dkv.norm", (m["kv_rank"],)), ("uk", (H * m["dim"], m["kv_rank"])),
+                            ("uv", (H * m["vdim"], m["kv_rank"])), ("g", (H * m["vdim"], w)), ("o", (w, H * m["vdim"]))):
+            out[n + "mix." + name] = shape
+        if layer["mlp"] is not None:
+            norm(n + "norm2")
+            norm(n + "norm2b")
+            ff = layer["mlp"]["ff"]
+            out[n + "mlp.gate"], out[n + "mlp.up"], out[n + "mlp.down"] = (ff, w), (ff, w), (w, ff)
+    norm("final.norm")
+    out["head"] = (config["vocab"], w)
+    return out
+
+
+def to_bf16(x) -> np.ndarray:
+    """float32 -> bfloat16 bits, to nearest even."""
+    u = np.ascontiguousarray(x, np.float32).view(np.uint32).astype(np.uint64)
+    return ((u + 0x7FFF + ((u >> 16) & 1)) >> 16).astype(np.uint16)
+
+
+def from_bf16(bits) -> np.ndarray:
+    return (np.asarray(bits, np.uint16).astype(np.uint32) << 16).view(np.float32)
+
+
+def vabirax_tensors(config, seed) -> dict:
+    """Random weights, bfloat16 bits by name: matrices with unit gain, norms that differ from element to element."""
+    rng = np.random.default_rng(seed)
+    out = {}
+    for name, shape in vabirax_shapes(config).items():
+        if len(shape) == 2:
+            v = rng.standard_normal(shape) * (1.0 if name == "embed" else shape[1] ** -0.5)
+        elif name.endswith(".alpha"):
+            v = rng.uniform(0.5, 1.2)
+        elif name.endswith(".b"):
+            v = rng.standard_normal(shape) * 0.1
+        else:
+            v = rng.uniform(0.5, 1.5, shape)
+        out[name] = to_bf16(np.asarray(v, np.float32)).reshape(shape)
+    return out
+
+
+def write_model_folder(path, config, tensors) -> None:
+    """config.json and model.safetensors; tensors: bfloat16 bits (uint16) or float32 arrays by name, or {name: (shape, function
+    that writes the bfloat16 bytes to a file)} for models that should not be held in memory."""
+    import json
+    import os
+    os.makedirs(path, exist_ok=True)
+    with open(os.path.join(path, "config.json"), "w") as f:
+        json.dump(config, f, indent=1)
+    header, at = {}, 0
+    for name, t in tensors.items():
+        shape, bits = (t[0], 16) if isinstance(t, tuple) else (t.shape, 16 if t.dtype == np.uint16 else 32)
+        n = int(np.prod(shape, dtype=np.int64)) * bits // 8
+        header[name] = {"dtype": "BF16" if bits == 16 else "F32", "shape": list(shape), "data_offsets": [at, at + n]}
+        at += n
+    text = json.dumps(header).encode()
+    text += b" " * (-len(text) % 8)
+    with open(os.path.join(path, "model.safetensors"), "wb") as f:
+        f.write(len(text).to_bytes(8, "little") + text)
+        for t in tensors.values():
+            if isinstance(t, tuple):
+                t[1](f)
+            else:
+                f.write(np.ascontiguousarray(t).tobytes())
+
+
+def vabirax_stream(config, seed) -> dict:
+    """Random weights for write_model_folder that are made while they are written: slices of one pool of normal numbers, scaled
+    by the power of two nearest to unit gain.  For timing at real sizes."""
+    rng = np.random.default_rng(seed)
+    pool = to_bf16(rng.standard_normal(1 << 22, dtype=np.float32))
+
+    def matrix(shape, shift):
+        def write(f):
+            left = int(np.prod(shape, dtype=np.int64))
+            while left:
+                a = int(rng.integers(0, pool.size // 2))
+                part = pool[a:a + min(left, pool.size - a)]
+                exp = (part >> 7) & 0xFF
+                f.write(np.where(exp > shift, part - np.uint16(shift << 7), np.uint16(0)).astype(np.uint16).tobytes())
+                left -= part.size
+        return write
+
+    out = {}
+    for name, shape in vabirax_shapes(config).items():
+        if len(shape) == 2:
+            out[name] = (shape, matrix(shape, 0 if name == "embed" else int(round(np.log2(shape[1]) / 2))))
+        else:
+            out[name] = to_bf16(np.full(shape, 0.7 if name.endswith(".alpha") else 0.0 if name.endswith(".b") else 1.0, np.float32)).reshape(shape)
+    return out
+
+
+def vabirax_1b() -> dict:
+    """Layers of Llama-3.2-1B's width, depth and feed-forward; 16 heads of 128 + 64 (values 128), latents of 768 and 512."""
+    layer = vabirax_layer(16, 128, 64, 128, 768, 512, 8192, 4096, base=500000.0)
+    return vabirax_config(2048, 128256, [layer] * 16, loop=(4, 12, 1), embedding_scale=1.0)
+
+
+def vabirax_3b() -> dict:
+    """Llama-3.2-3B's width, depth and feed-forward; 24 heads of 128 + 64 (values 128), latents of 1536 and 512."""
+    layer = vabirax_layer(24, 128, 64, 128, 1536, 512, 8192, 4096, base=500000.0)
+    return vabirax_config(3072, 128256, [layer] * 28, loop=(8, 20, 1), embedding_scale=1.0)
