@@ -468,6 +468,9 @@ def vabirax_bench(fh, args):
     line["decode_other_us"] = {s: round(v[0], 1) for s, v in dec.items() if s not in dec_bytes and v[1]}
     line["prefill_other_ms"] = {s: round(v[0], 3) for s, v in pre.items() if s not in pre_ops and v[1]}
 
+    if args.no_closest:
+        print(js.dumps({"vabirax": line}))
+        return
     lcfg = getattr(fh.synth, "llama32_" + args.vabirax)(fh.Q8_0, max_seq=max_seq)
     blob = fh.synth.make_weights_blob(lcfg, seed=args.seed, threads=16)
     print("Llama weights made", file=sys.stderr, flush=True)
@@ -518,6 +521,7 @@ def main():
                     help="length of the prompt (default: the 2502 tokens the metric is quoted on); the cache is sized to fit")
     ap.add_argument("--ops-table", action="store_true",
                     help="instead of the model benchmark, run the isolated kernels at the benchmark configurations' sizes")
+    ap.add_argument("--no-closest", action="store_true", help="with --vabirax: skip the Llama-family model")
     ap.add_argument("--vabirax", choices=("1b", "3b"),
                     help="instead of the default workload, the Vabirax design at this size beside the Llama-family model of the same size")
     args = ap.parse_args()

@@ -44,7 +44,7 @@ EXPORTS = [
     "forge_hip_gguf_config_mixed", "forge_hip_gguf_export_weights_mixed", "forge_hip_quantize_kquant",
     "forge_hip_model_create_from_gguf", "forge_hip_dequant_ggml", "forge_hip_model_set_repeat_penalty", "forge_hip_apply_repeat_penalty", "forge_hip_sample",
     "forge_hip_prefill_logits", "forge_hip_model_create_from_folder", "forge_hip_folder_config", "forge_hip_model_config",
-    "forge_hip_model_layer_runs", "forge_hip_prefill_residuals",
+    "forge_hip_model_layer_runs", "forge_hip_prefill_residuals", "forge_hip_dense_matmul",
 ]
 
 
@@ -174,6 +174,8 @@ def lib():
     L.forge_hip_attn_prefill_sliding_f16kv.argtypes = [vp, vp, vp, vp, u32, u32, u32, u32, u32, u32, u32, vp]
     L.forge_hip_attn_decode_sliding_f16kv.restype = i32
     L.forge_hip_attn_decode_sliding_f16kv.argtypes = [vp, vp, vp, vp, u32, u32, u32, u32, u32, u32, vp]
+    L.forge_hip_dense_matmul.restype = i32
+    L.forge_hip_dense_matmul.argtypes = [u32, vp, vp, u32, u32, u32, vp, vp]
     L.forge_hip_argmax.restype = i32
     L.forge_hip_argmax.argtypes = [vp, u32, vp, vp]
     L.forge_hip_model_set_repeat_penalty.restype = i32

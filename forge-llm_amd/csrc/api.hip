@@ -449,6 +449,23 @@ int32_t forge_hip_expf_host(const float* x_host, uint64_t n, float* out_host) {
     return FORGE_HIP_OK;
 }
 
+int32_t forge_hip_dense_matmul(uint32_t dtype, const void* w_dev, const void* a_dev, uint32_t M, uint32_t N, uint32_t K, float* y_dev, void* stream) {
+    FH_CHECK(dtype == FORGE_HIP_BF16 || dtype == FORGE_HIP_F32, "dense_matmul: dtype must be BF16 (30) or F32 (0)");
+    FH_CHECK(w_dev && a_dev && y_dev, "dense_matmul: null pointer");
+    FH_CHECK(M >= 1 && N >= 1, "dense_matmul: M and N must be positive");
+    FH_CHECK(K >= 64 && K % 64 == 0 && K <= dense_k_max(), "dense_matmul: K must be a multiple of 64, at most 32768");
+    DenseWeight w;
+    w.p = const_cast<void*>(w_dev);
+    w.N = N;
+    w.K = K;
+    DenseEpiArgs e;
+    e.f32 = y_dev;
+    e.ld_f32 = N;
+    launch_dense((DType)dtype, w, a_dev, K, M, DenseEpi::F32, e, (hipStream_t)stream);
+    FH_HIP(hipGetLastError());
+    return FORGE_HIP_OK;
+}
+
 int32_t forge_hip_argmax(const float* x_dev, uint32_t n, uint32_t* out_dev, void* stream) {
     FH_CHECK(x_dev && out_dev && n >= 1, "argmax: null pointer or empty input");
     int32_t rc = g_attn.reserve(ARGMAX_BLOCKS * 8);

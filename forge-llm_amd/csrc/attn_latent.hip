@@ -17,7 +17,8 @@
 namespace fh {
 
 constexpr float LOG2E = 1.4426950408889634f;
-constexpr uint32_t RANK_MAX = 1024, HEAD_DIM_MAX = 256, SPLITS_MAX = 32;
+constexpr float NO_KEYS = -3.0e38f;          // maximum of a part without keys: weight 0, and finite where another layer's records overlap it
+constexpr uint32_t RANK_MAX = 1024, HEAD_DIM_MAX = 256, SPLITS_MAX = 64;
 
 // ---- the new cache row and the normed query latent of one position; `tid` of `nt` threads, red: LDS, nt / 64 floats -----------------
 __device__ __forceinline__ float block_sum(float v, float* red, uint32_t tid, uint32_t nt) {
@@ -68,33 +69,43 @@ __global__ __launch_bounds__(256) void latent_norm_store_kernel(LatentShape sh, 
 }
 
 // ---- prompt ---------------------------------------------------------------------------------------------------------------
-// Workgroup = 4 waves = 128 consecutive queries of one head, 32 per wave; keys and values stream through LDS in tiles of 64
-// (K row-major: unrotated part, rotated part; V transposed), the next tile's loads in registers while this one is worked.  Both
-// products are computed transposed (S^T = K Q^T, O^T = V^T P^T): a lane owns one query, so the softmax statistics are per-lane
-// scalars, and the exponentiated scores are already the second product's operand.  Scores stay in the base-2 domain.
+// Workgroup = 8 waves = 128 consecutive queries of one head: four groups of 32, each shared by two waves that take one half
+// (32 keys) of every key tile and merge their (maximum, sum, output) at the end, which halves the longest chain of dependent
+// tile steps.  Keys and values stream through LDS in tiles of 64 (K row-major: unrotated part, rotated part; V transposed), the
+// next tile's loads in registers while this one is worked.  Both products are computed transposed (S^T = K Q^T, O^T = V^T P^T):
+// a lane owns one query, so the softmax statistics are per-lane scalars, and the exponentiated scores are already the second
+// product's operand.  Scores stay in the base-2 domain.
 // DQ >= dim + rot and DV >= vdim: the register tiles' sizes; columns past the real ones are zero.
+constexpr uint32_t LP_KT = 64, LP_QB = 128, LP_THREADS = 512;
+template <typename T, int DQ, int DV> constexpr uint32_t latent_prefill_lds() {
+    const uint32_t tiles = (LP_KT * (DQ + 16 / sizeof(T)) + DV * (LP_KT + 8 / sizeof(T))) * sizeof(T), merge = 4 * 64 * 18 * 4;
+    return tiles > merge ? tiles : merge;
+}
+
 template <typename T, int DQ, int DV>
-__global__ __launch_bounds__(256) void latent_attn_prefill_kernel(LatentShape sh, const T* __restrict__ q, const T* __restrict__ kbuf, const T* __restrict__ vbuf,
-                                                                  const T* __restrict__ cache, uint32_t kv_lo, const T* __restrict__ gate, T* __restrict__ out,
-                                                                  uint32_t ld_out, uint32_t M, uint32_t base_pos) {
+__global__ __launch_bounds__(LP_THREADS) __attribute__((amdgpu_waves_per_eu(2)))
+void latent_attn_prefill_kernel(LatentShape sh, const T* __restrict__ q, const T* __restrict__ kbuf, const T* __restrict__ vbuf,
+                                const T* __restrict__ cache, uint32_t kv_lo, const T* __restrict__ gate, T* __restrict__ out,
+                                uint32_t ld_out, uint32_t M, uint32_t base_pos) {
     typedef typename Vec<T>::x4 x4;
     typedef typename Vec<T>::x8 x8;
-    constexpr uint32_t KT = 64, QB = 128, PAD = 16 / sizeof(T);
+    constexpr uint32_t KT = LP_KT, QB = LP_QB, NT = LP_THREADS, PAD = 16 / sizeof(T);
     constexpr uint32_t KS = DQ + PAD, VS = KT + 8 / sizeof(T);         // LDS row strides
     constexpr uint32_t NS = DQ / 16, ND = DV / 32;
-    constexpr uint32_t KP = KT * DQ / 8 / 256, VP = (KT / 2) * (DV / 4) / 256;
-    static_assert(KT * DQ / 8 % 256 == 0 && (KT / 2) * (DV / 4) % 256 == 0, "whole pieces per thread");
+    constexpr uint32_t KTOTAL = KT * DQ / 8, VTOTAL = (KT / 2) * (DV / 4);       // pieces of a tile
+    constexpr uint32_t KP = (KTOTAL + NT - 1) / NT, VP = (VTOTAL + NT - 1) / NT;
     extern __shared__ __attribute__((aligned(16))) uint8_t lat_lds[];
     T* Ks = reinterpret_cast<T*>(lat_lds);
     T* Vt = Ks + KT * KS;
 
     const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, lq = lane & 31, lh = lane >> 5;
+    const uint32_t qg = wave >> 1, kh = wave & 1;        // query group, half of every key tile
     // latest (longest) query tiles first
     const uint32_t head = blockIdx.x % sh.heads, ntq = gridDim.x / sh.heads;
     const uint32_t q0 = (ntq - 1 - blockIdx.x / sh.heads) * QB;
     const uint32_t dq = sh.dim + sh.rot, window = sh.window ? sh.window : 0xFFFFFFFFu;
     const float c2 = sh.scale * LOG2E;
-    const uint32_t qrow = q0 + wave * 32 + lq, qpos = base_pos + qrow;
+    const uint32_t qrow = q0 + qg * 32 + lq, qpos = base_pos + qrow;
 
     x8 qf[NS];
 #pragma unroll
@@ -111,10 +122,10 @@ __global__ __launch_bounds__(256) void latent_attn_prefill_kernel(LatentShape sh
 
     const uint32_t total = base_pos + M;
     const uint32_t wg_max = base_pos + min(q0 + QB, M) - 1, wg_min = base_pos + q0;
-    const bool wave_active = q0 + wave * 32 < M;
-    const uint32_t wave_min = wg_min + wave * 32, wave_max = base_pos + min(q0 + wave * 32 + 32, M) - 1;
+    const bool wave_active = q0 + qg * 32 < M;
+    const uint32_t wave_min = wg_min + qg * 32, wave_max = base_pos + min(q0 + qg * 32 + 32, M) - 1;
     auto first_visible = [&](uint32_t p) { return p >= window ? p - window + 1 : 0u; };
-    const uint32_t wave_lo = first_visible(wave_min);
+    const uint32_t wave_lo = first_visible(wave_min), last_lo = first_visible(wave_max);
     const uint32_t tile0 = first_visible(wg_min) / KT, ntiles = wg_max / KT + 1;
 
     const uint32_t kst = sh.heads * sh.dim, vst = sh.heads * sh.vdim, cst = sh.cache_row();
@@ -123,16 +134,16 @@ __global__ __launch_bounds__(256) void latent_attn_prefill_kernel(LatentShape sh
     auto load_tile = [&](uint32_t kt) {
 #pragma unroll
         for (uint32_t i = 0; i < KP; i++) {
-            const uint32_t idx = tid + 256 * i, key = idx / (DQ / 8), d = idx % (DQ / 8) * 8, t = kt * KT + key;
-            if (t >= total || d >= dq) kreg[i] = zero8<T>();
+            const uint32_t idx = tid + NT * i, key = idx / (DQ / 8), d = idx % (DQ / 8) * 8, t = kt * KT + key;
+            if (idx >= KTOTAL || t >= total || d >= dq) kreg[i] = zero8<T>();
             else kreg[i] = d < sh.dim ? load8(kbuf + (size_t)(t - kv_lo) * kst + head * sh.dim + d)
                                       : load8(cache + (size_t)t * cst + sh.rank + (d - sh.dim));
         }
 #pragma unroll
         for (uint32_t i = 0; i < VP; i++) {
-            const uint32_t idx = tid + 256 * i, kp = idx / (DV / 4), d = idx % (DV / 4) * 4, t = kt * KT + 2 * kp;
+            const uint32_t idx = tid + NT * i, kp = idx / (DV / 4), d = idx % (DV / 4) * 4, t = kt * KT + 2 * kp;
             const T* src = vbuf + (size_t)(t - kv_lo) * vst + head * sh.vdim + d;
-            const bool in = d < sh.vdim;
+            const bool in = idx < VTOTAL && d < sh.vdim;
             x4 z;
 #pragma unroll
             for (int e = 0; e < 4; e++) z[e] = (T)0.f;
@@ -143,13 +154,14 @@ __global__ __launch_bounds__(256) void latent_attn_prefill_kernel(LatentShape sh
     auto store_tile = [&]() {
 #pragma unroll
         for (uint32_t i = 0; i < KP; i++) {
-            const uint32_t idx = tid + 256 * i, key = idx / (DQ / 8), d = idx % (DQ / 8) * 8;
-            store8(Ks + key * KS + d, kreg[i]);
+            const uint32_t idx = tid + NT * i, key = idx / (DQ / 8), d = idx % (DQ / 8) * 8;
+            if (idx < KTOTAL) store8(Ks + key * KS + d, kreg[i]);
         }
         // the two keys' values of one column side by side
 #pragma unroll
         for (uint32_t i = 0; i < VP; i++) {
-            const uint32_t idx = tid + 256 * i, kp = idx / (DV / 4), d = idx % (DV / 4) * 4;
+            const uint32_t idx = tid + NT * i, kp = idx / (DV / 4), d = idx % (DV / 4) * 4;
+            if (idx >= VTOTAL) continue;
 #pragma unroll
             for (int e = 0; e < 4; e++) {
                 struct __attribute__((aligned(2 * sizeof(T)))) Pair { T a, b; } p = {va[i][e], vb[i][e]};
@@ -164,36 +176,30 @@ __global__ __launch_bounds__(256) void latent_attn_prefill_kernel(LatentShape sh
         store_tile();
         __syncthreads();
         if (kt + 1 < ntiles) load_tile(kt + 1);
-        const uint32_t k0 = kt * KT;
-        if (!(wave_active && k0 <= wave_max && k0 + KT > wave_lo)) continue;       // all in the wave's future, or before its windows
-        v16f sacc[2];
+        const uint32_t k0 = kt * KT + kh * 32;                                     // the wave's 32 keys
+        if (!(wave_active && k0 <= wave_max && k0 + 32 > wave_lo)) continue;       // all in the wave's future, or before its windows
+        // two accumulators: a product waits for the one before the last
+        v16f sacc, sodd;
 #pragma unroll
-        for (int h = 0; h < 2; h++)
+        for (int r = 0; r < 16; r++) sacc[r] = sodd[r] = 0.f;
 #pragma unroll
-            for (int r = 0; r < 16; r++) sacc[h][r] = 0.f;
+        for (uint32_t s = 0; s < NS; s += 2) {
+            sacc = mma32(load8(Ks + (kh * 32 + lq) * KS + 16 * s + 8 * lh), qf[s], sacc);
+            sodd = mma32(load8(Ks + (kh * 32 + lq) * KS + 16 * (s + 1) + 8 * lh), qf[s + 1], sodd);
+        }
+        if (k0 + 31 > wave_min || k0 < last_lo) {
 #pragma unroll
-        for (uint32_t s = 0; s < NS; s++)
-#pragma unroll
-            for (int h = 0; h < 2; h++) sacc[h] = mma32(load8(Ks + (h * 32 + lq) * KS + 16 * s + 8 * lh), qf[s], sacc[h]);
-        if (k0 + KT - 1 > wave_min || (sh.window && k0 < first_visible(wave_max))) {
-#pragma unroll
-            for (int h = 0; h < 2; h++)
-#pragma unroll
-                for (int r = 0; r < 16; r++) {
-                    const uint32_t t = k0 + 32 * h + 8 * (r >> 2) + 4 * lh + (r & 3);
-                    sacc[h][r] = (t <= qpos && qpos - t < window) ? sacc[h][r] * c2 : -INFINITY;
-                }
+            for (int r = 0; r < 16; r++) {
+                const uint32_t t = k0 + 8 * (r >> 2) + 4 * lh + (r & 3);
+                sacc[r] = (t <= qpos && qpos - t < window) ? (sacc[r] + sodd[r]) * c2 : -INFINITY;
+            }
         } else {
 #pragma unroll
-            for (int h = 0; h < 2; h++)
-#pragma unroll
-                for (int r = 0; r < 16; r++) sacc[h][r] *= c2;
+            for (int r = 0; r < 16; r++) sacc[r] = (sacc[r] + sodd[r]) * c2;
         }
-        float m_tile = -INFINITY;
+        float m_tile = sacc[0];
 #pragma unroll
-        for (int h = 0; h < 2; h++)
-#pragma unroll
-            for (int r = 0; r < 16; r++) m_tile = fmaxf(m_tile, sacc[h][r]);
+        for (int r = 1; r < 16; r++) m_tile = fmaxf(m_tile, sacc[r]);
         const float m_new = fmaxf(m_run, lane_xor_max<32>(m_tile));
         const float m_exp = m_new == -INFINITY ? 0.f : m_new;            // no key seen yet: every weight is 2^-inf = 0
         if (__builtin_amdgcn_ballot_w64(m_new > m_run) != 0) {
@@ -205,40 +211,57 @@ __global__ __launch_bounds__(256) void latent_attn_prefill_kernel(LatentShape sh
                 for (int r = 0; r < 16; r++) oacc[d][r] *= alpha;
         }
         m_run = m_new;
+        x8 pb[2];
 #pragma unroll
-        for (int h = 0; h < 2; h++)
+        for (int j = 0; j < 2; j++)
 #pragma unroll
-            for (int j = 0; j < 2; j++) {
-                x8 pb;
+            for (int e = 0; e < 8; e++) {
+                const float p = __builtin_amdgcn_exp2f(sacc[8 * j + e] - m_exp);
+                l_run += p;
+                pb[j][e] = (T)p;
+            }
+        // element e of lane half lh is key 16 j + 8 (e / 4) + 4 lh + e % 4 of the wave's half
 #pragma unroll
-                for (int e = 0; e < 8; e++) {
-                    const float p = __builtin_amdgcn_exp2f(sacc[h][8 * j + e] - m_exp);
-                    l_run += p;
-                    pb[e] = (T)p;
-                }
-                // element e of lane half lh is key 32 h + 16 j + 8 (e / 4) + 4 lh + e % 4
+        for (int j = 0; j < 2; j++)
 #pragma unroll
-                for (uint32_t d = 0; d < ND; d++) {
-                    const T* vr = Vt + (d * 32 + lq) * VS + h * 32 + 16 * j + 4 * lh;
-                    const x4 v0 = *reinterpret_cast<const x4*>(vr), v1 = *reinterpret_cast<const x4*>(vr + 8);
-                    oacc[d] = mma32((x8){v0[0], v0[1], v0[2], v0[3], v1[0], v1[1], v1[2], v1[3]}, pb, oacc[d]);
-                }
+            for (uint32_t d = 0; d < ND; d++) {
+                const T* vr = Vt + (d * 32 + lq) * VS + kh * 32 + 16 * j + 4 * lh;
+                const x4 v0 = *reinterpret_cast<const x4*>(vr), v1 = *reinterpret_cast<const x4*>(vr + 8);
+                oacc[d] = mma32((x8){v0[0], v0[1], v0[2], v0[3], v1[0], v1[1], v1[2], v1[3]}, pb[j], oacc[d]);
             }
     }
-    const float l_tot = lane_xor_add<32>(l_run);
-    if (qrow >= M) return;
-    const float inv = 1.0f / l_tot;
+
+    // ---- merge: the odd wave of a group hands its state over through LDS, 32 output columns at a time
+    float* mg = reinterpret_cast<float*>(lat_lds) + (qg * 64 + lane) * 18;
+    __syncthreads();
+    if (kh) { mg[16] = m_run; mg[17] = l_run; }
+    __syncthreads();
+    const float m1 = mg[16], l1 = mg[17], m_all = fmaxf(m_run, m1);       // finite for rows < M: a query sees itself
+    const float m_ref = m_all == -INFINITY ? 0.f : m_all;
+    const float a0 = __builtin_amdgcn_exp2f(m_run - m_ref), a1 = __builtin_amdgcn_exp2f(m1 - m_ref);
+    const float inv = 1.0f / lane_xor_add<32>(l_run * a0 + l1 * a1);
 #pragma unroll
-    for (uint32_t d = 0; d < ND; d++)
+    for (uint32_t d = 0; d < ND; d++) {
+        if (kh) {
 #pragma unroll
-        for (int g = 0; g < 4; g++) {
-            const uint32_t c = 32 * d + 8 * g + 4 * lh;
-            if (c >= sh.vdim) continue;
-            const size_t at = (size_t)qrow * ld_out + head * sh.vdim + c;
-            const x4 gt = *reinterpret_cast<const x4*>(gate + at);
-            store4<T>(out + at, oacc[d][4 * g] * inv * (float)gt[0], oacc[d][4 * g + 1] * inv * (float)gt[1], oacc[d][4 * g + 2] * inv * (float)gt[2],
-                      oacc[d][4 * g + 3] * inv * (float)gt[3]);
+            for (int r = 0; r < 16; r++) mg[r] = oacc[d][r];
         }
+        __syncthreads();
+        if (!kh && qrow < M) {
+#pragma unroll
+            for (int g = 0; g < 4; g++) {
+                const uint32_t c = 32 * d + 8 * g + 4 * lh;
+                if (c >= sh.vdim) continue;
+                const size_t at = (size_t)qrow * ld_out + head * sh.vdim + c;
+                const x4 gt = *reinterpret_cast<const x4*>(gate + at);
+                float o[4];
+#pragma unroll
+                for (int i = 0; i < 4; i++) o[i] = (oacc[d][4 * g + i] * a0 + mg[4 * g + i] * a1) * inv * (float)gt[i];
+                store4<T>(out + at, o[0], o[1], o[2], o[3]);
+            }
+        }
+        __syncthreads();
+    }
 }
 
 // ---- decode ----------------------------------------------------------------------------------------------------------------
@@ -301,6 +324,7 @@ __global__ __launch_bounds__(NW * 64) void latent_attn_decode_kernel(LatentShape
     constexpr uint32_t KT = 16 * NW, PAD = 16 / sizeof(T), VS = KT + PAD;
     constexpr uint32_t KSTEPS = KT / 32;
     static_assert(KT % 32 == 0, "the second product works 32 keys at a time");
+    static_assert(SPLITS_MAX == 64, "the parts' weights are made by one wave");
     extern __shared__ __attribute__((aligned(16))) uint8_t ld_lds[];
     T* Ct = reinterpret_cast<T*>(ld_lds);                   // [rank][VS]
     T* P = Ct + sh.rank * VS;                               // [16][VS]
@@ -347,21 +371,28 @@ __global__ __launch_bounds__(NW * 64) void latent_attn_decode_kernel(LatentShape
                 for (int e = 0; e < 8; e++) Ct[(32 * s + 8 * lg + e) * VS + 16 * wave + l16] = f[e];
             }
         };
-        constexpr uint32_t U = sizeof(T) == 2 ? 4 : 2;
-        uint32_t s = 0;
-        for (; s + U <= NSR; s += U) {
+        // bfloat16: a whole row of up to 512 latents is requested at once, with the first rotated dimensions
+        constexpr uint32_t U = sizeof(T) == 2 ? (MAXT * NW / 2 < 16 ? MAXT * NW / 2 : 16) : 2;
+        constexpr uint32_t UR = 2;
+        x8 fr[UR], gr[UR];
+#pragma unroll
+        for (uint32_t u = 0; u < UR; u++) {
+            const bool in = NSR + u < NS;
+            fr[u] = in ? load8(row + 32 * (NSR + u)) : zero8<T>();
+            gr[u] = in ? load8(qr + 32 * u) : zero8<T>();
+        }
+        for (uint32_t s = 0; s < NSR; s += U) {
             x8 f[U], g[U];
 #pragma unroll
-            for (uint32_t u = 0; u < U; u++) { f[u] = load8(row + 32 * (s + u)); g[u] = load8(qn + 32 * (s + u)); }
+            for (uint32_t u = 0; u < U; u++)
+                if (s + u < NSR) { f[u] = load8(row + 32 * (s + u)); g[u] = load8(qn + 32 * (s + u)); }
 #pragma unroll
-            for (uint32_t u = 0; u < U; u++) { sacc = mma16(f[u], g[u], sacc); lay_down(s + u, f[u]); }
+            for (uint32_t u = 0; u < U; u++)
+                if (s + u < NSR) { sacc = mma16(f[u], g[u], sacc); lay_down(s + u, f[u]); }
         }
-        for (; s < NSR; s++) {
-            const x8 f = load8(row + 32 * s);
-            sacc = mma16(f, load8(qn + 32 * s), sacc);
-            lay_down(s, f);
-        }
-        for (; s < NS; s++) sacc = mma16(load8(row + 32 * s), load8(qr + 32 * (s - NSR)), sacc);
+#pragma unroll
+        for (uint32_t u = 0; u < UR; u++) sacc = mma16(fr[u], gr[u], sacc);
+        for (uint32_t s = NSR + UR; s < NS; s++) sacc = mma16(load8(row + 32 * s), load8(qr + 32 * (s - NSR)), sacc);
         // register r: key tk + 4 lg + r, this lane's head
         float mx = -INFINITY;
 #pragma unroll
@@ -411,37 +442,54 @@ __global__ __launch_bounds__(NW * 64) void latent_attn_decode_kernel(LatentShape
         if (tid < 16) {
             float l = 0.f;
             for (int w = 0; w < NW; w++) l += smax[w * 16 + l16];
-            rec[sh.rank] = m_run;                  // -inf: an empty part, whose sums are not read
+            rec[sh.rank] = t0 < t1 ? m_run : NO_KEYS;
             rec[sh.rank + 1] = l;
         }
     }
 }
 
 // [merge of the parts | W_uv | gate]: a workgroup's rows belong to one head.
-template <typename T, int KS>
+template <typename T>
 __global__ __launch_bounds__(GEMV_THREADS) void latent_value_kernel(LatentShape sh, const float* __restrict__ parts, uint32_t nparts, const T* __restrict__ uv, DenseEpiArgs e) {
     extern __shared__ __attribute__((aligned(16))) float lv_lds[];
-    const uint32_t tid = threadIdx.x, K = sh.rank, row0 = blockIdx.x * gemv_rows<KS>();
-    const uint32_t head = row0 / sh.vdim;
+    // the workgroups of a head are `heads` apart: with a multiple of 8 heads they sit on one XCD and share the parts in its L2
+    const uint32_t tid = threadIdx.x, K = sh.rank, head = blockIdx.x % sh.heads;
+    const uint32_t row0 = head * sh.vdim + blockIdx.x / sh.heads * gemv_rows<1>();
     float* xs = lv_lds;
     float* red = lv_lds + K;
     float* wt = red + 16;           // [SPLITS_MAX]
-    gemv_body<T, KS, DenseEpi::GateMul>(uv, sh.heads * sh.vdim, K, row0, xs, red, e, [&]() {
+    gemv_body<T, 1, DenseEpi::GateMul>(uv, sh.heads * sh.vdim, K, row0, xs, red, e, [&]() {
         const size_t step = (size_t)sh.heads * (sh.rank + 4);
         const float* rec = parts + (size_t)head * (sh.rank + 4);
+        // the first sums are requested ahead of the statistics they are weighted with
+        constexpr uint32_t B = 32;
+        float2 r[B];
+        auto fetch = [&](uint32_t p0, uint32_t i) {
+#pragma unroll
+            for (uint32_t p = 0; p < B; p++) r[p] = *reinterpret_cast<const float2*>(rec + min(p0 + p, nparts - 1) * step + i);
+        };
+        if (tid * 2 < K) fetch(0, tid * 2);
         if (tid < 64) {
             const float m = tid < nparts ? rec[tid * step + sh.rank] : -INFINITY;
+            const float ls = tid < nparts ? rec[tid * step + sh.rank + 1] : 0.f;
             const float mx = wave_max(m);
-            const float w = m == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m - mx);
-            const float l = wave_sum(w > 0.f ? w * rec[tid * step + sh.rank + 1] : 0.f);
-            if (tid < SPLITS_MAX) wt[tid] = w / l;
+            const float w = __builtin_amdgcn_exp2f(m - mx);          // mx is finite: some part holds keys
+            const float l = wave_sum(w * ls);
+            wt[tid] = w / l;                                         // 0 past the last part
         }
         __syncthreads();
-        for (uint32_t i = tid; i < K; i += GEMV_THREADS) {
-            float v = 0.f;
-            for (uint32_t p = 0; p < nparts; p++)
-                if (wt[p] > 0.f) v = fmaf(wt[p], rec[p * step + i], v);
-            xs[i] = v;
+        for (uint32_t i = tid * 2; i < K; i += GEMV_THREADS * 2) {
+            float v0 = 0.f, v1 = 0.f;
+            for (uint32_t p0 = 0; p0 < nparts; p0 += B) {
+                if (p0 || i != tid * 2) fetch(p0, i);
+#pragma unroll
+                for (uint32_t p = 0; p < B; p++) {
+                    v0 = fmaf(wt[p0 + p], r[p].x, v0);
+                    v1 = fmaf(wt[p0 + p], r[p].y, v1);
+                }
+            }
+            xs[i] = v0;
+            xs[i + 1] = v1;
         }
     });
 }
@@ -451,12 +499,12 @@ namespace {
 template <typename T, int DQ, int DV>
 void go_prefill(const LatentShape& sh, const void* q, const void* kbuf, const void* vbuf, const void* cache, uint32_t kv_lo, const void* gate,
                 void* out, uint32_t ld_out, uint32_t M, uint32_t base_pos, hipStream_t s) {
-    constexpr uint32_t lds = (64 * (DQ + 16 / sizeof(T)) + DV * (64 + 8 / sizeof(T))) * sizeof(T);
+    constexpr uint32_t lds = latent_prefill_lds<T, DQ, DV>();
     static_assert(lds <= 160 * 1024, "LDS of a compute unit");
     static const hipError_t ok = hipFuncSetAttribute((const void*)latent_attn_prefill_kernel<T, DQ, DV>, hipFuncAttributeMaxDynamicSharedMemorySize, lds);
     (void)ok;
-    fh::launch(latent_attn_prefill_kernel<T, DQ, DV>, dim3((M + 127) / 128 * sh.heads), 256, lds, s, sh, (const T*)q, (const T*)kbuf, (const T*)vbuf,
-               (const T*)cache, kv_lo, (const T*)gate, (T*)out, ld_out, M, base_pos);
+    fh::launch(latent_attn_prefill_kernel<T, DQ, DV>, dim3((M + LP_QB - 1) / LP_QB * sh.heads), LP_THREADS, lds, s, sh, (const T*)q, (const T*)kbuf,
+               (const T*)vbuf, (const T*)cache, kv_lo, (const T*)gate, (T*)out, ld_out, M, base_pos);
 }
 
 template <typename T>
@@ -524,11 +572,10 @@ void decode(const LatentShape& sh, const LatentDecodeIo& io, hipStream_t s) {
     DenseEpiArgs e;
     e.out = io.out;
     e.gate = io.gate;
-    // rows of a workgroup (16 or 4) lie in one head: vdim is a multiple of 32
+    // the 16 rows of a workgroup lie in one head (vdim is a multiple of 32); every workgroup merges its head's parts, so few of them
     const T* uv = (const T*)io.ukv.p + (size_t)sh.heads * sh.dim * sh.rank;
     const uint32_t N = sh.heads * sh.vdim, lds = (sh.rank + 16 + SPLITS_MAX) * 4, np = latent_splits(sh, io.max_seq);
-    if (gemv_depth_split(N, sh.rank) == 1) fh::launch(latent_value_kernel<T, 1>, dim3(N / gemv_rows<1>()), GEMV_THREADS, lds, s, sh, io.parts, np, uv, e);
-    else fh::launch(latent_value_kernel<T, 4>, dim3(N / gemv_rows<4>()), GEMV_THREADS, lds, s, sh, io.parts, np, uv, e);
+    fh::launch(latent_value_kernel<T>, dim3(N / gemv_rows<1>()), GEMV_THREADS, lds, s, sh, io.parts, np, uv, e);
 }
 
 }  // namespace

@@ -402,6 +402,8 @@ int32_t BlockModel::alloc_scratch() {
         (rc = parts.alloc(pb)) || (rc = rows_sel.alloc(HEAD_ROWS * 4)) || (rc = h_sel.alloc(HEAD_ROWS * width * es)))
         return rc;
     if (loop_in.p && (rc = xcat.alloc(R * 2 * width * es))) return rc;
+    // parts without keys keep what they held: weighted with 0, which needs a finite number
+    FH_HIP(hipMemset(parts.p, 0, pb));
     // columns that pad the concatenated heads are read (against zero weights) and never written
     FH_HIP(hipMemset(attn.p, 0, R * hv * es));
     return FORGE_HIP_OK;

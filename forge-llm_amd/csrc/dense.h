@@ -111,17 +111,24 @@ __device__ __forceinline__ void dense_epilogue(const DenseEpiArgs& e, uint32_t m
         y[0] = (T)(silu_f(v[0]) * v[1]);
         y[1] = (T)(silu_f(v[2]) * v[3]);
     } else if constexpr (MODE == DenseEpi::Residual) {
+        // everything the four results need is requested at once
         float4* xp = reinterpret_cast<float4*>(e.f32 + (size_t)m * e.ld_f32 + n);
-        float a[4];
-#pragma unroll
-        for (int i = 0; i < 4; i++) a[i] = dyn_tanh(e.post, n + i, v[i]);
-        if (e.add) {
-            const float4 x = *xp;
-            a[0] += x.x; a[1] += x.y; a[2] += x.z; a[3] += x.w;
-        }
+        const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f);
+        const float4 x = e.add ? *xp : zero;
+        const float4 pw = e.post.w ? *reinterpret_cast<const float4*>(e.post.w + n) : zero, pb = e.post.w ? *reinterpret_cast<const float4*>(e.post.b + n) : zero;
+        const float4 nw = e.next.w ? *reinterpret_cast<const float4*>(e.next.w + n) : zero, nb = e.next.w ? *reinterpret_cast<const float4*>(e.next.b + n) : zero;
+        float a[4] = {v[0], v[1], v[2], v[3]};
+        auto norm4 = [&](const DynTanh& t, const float4& w, const float4& b) {
+            if (!t.w) return;
+            a[0] = tanhf(t.alpha * a[0]) * w.x + b.x;
+            a[1] = tanhf(t.alpha * a[1]) * w.y + b.y;
+            a[2] = tanhf(t.alpha * a[2]) * w.z + b.z;
+            a[3] = tanhf(t.alpha * a[3]) * w.w + b.w;
+        };
+        norm4(e.post, pw, pb);
+        a[0] += x.x; a[1] += x.y; a[2] += x.z; a[3] += x.w;
         *xp = make_float4(a[0], a[1], a[2], a[3]);
-#pragma unroll
-        for (int i = 0; i < 4; i++) a[i] = dyn_tanh(e.next, n + i, a[i]);
+        norm4(e.next, nw, nb);
         store4<T>((T*)e.out + (size_t)m * e.ld_out + n, a[0], a[1], a[2], a[3]);
     }
 }

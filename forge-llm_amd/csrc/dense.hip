@@ -133,14 +133,14 @@ template <typename T>
 __global__ __launch_bounds__(256) void dense_embedding_kernel(const T* __restrict__ table, uint32_t width, float scale, const uint32_t* __restrict__ tokens,
                                                               float* __restrict__ x, uint32_t ldx, DynTanh next, T* __restrict__ out, uint32_t ld_out,
                                                               T* __restrict__ out2, uint32_t ld_out2, uint32_t* __restrict__ counts) {
-    const uint32_t m = blockIdx.x, tok = tokens[m];
-    for (uint32_t i = threadIdx.x; i < ldx; i += blockDim.x) {
+    const uint32_t m = blockIdx.y, tok = tokens[m], i = blockIdx.x * 256 + threadIdx.x;
+    if (i < ldx) {
         const float v = i < width ? (float)table[(size_t)tok * width + i] * scale : 0.f;
         x[(size_t)m * ldx + i] = v;
         out[(size_t)m * ld_out + i] = (T)dyn_tanh(next, i, v);
         if (out2) out2[(size_t)m * ld_out2 + i] = (T)v;
     }
-    if (threadIdx.x == 0 && counts) atomicAdd(counts + tok, 1u);
+    if (i == 0 && counts) atomicAdd(counts + tok, 1u);
 }
 
 template <typename T>
@@ -212,10 +212,10 @@ void launch_dense(DType t, const DenseWeight& w, const void* a, uint32_t lda, ui
 void launch_dense_embedding(DType t, const void* table, uint32_t width, float scale, const uint32_t* tokens_dev, uint32_t M, float* x,
                             uint32_t ldx, const DynTanh& next, void* out, uint32_t ld_out, void* out2, uint32_t ld_out2, uint32_t* counts, hipStream_t s) {
     if (t == DType::BF16)
-        fh::launch(dense_embedding_kernel<__bf16>, dim3(M), 256, 0, s, (const __bf16*)table, width, scale, tokens_dev, x, ldx, next, (__bf16*)out, ld_out,
+        fh::launch(dense_embedding_kernel<__bf16>, dim3((ldx + 255) / 256, M), 256, 0, s, (const __bf16*)table, width, scale, tokens_dev, x, ldx, next, (__bf16*)out, ld_out,
                    (__bf16*)out2, ld_out2, counts);
     else
-        fh::launch(dense_embedding_kernel<float>, dim3(M), 256, 0, s, (const float*)table, width, scale, tokens_dev, x, ldx, next, (float*)out, ld_out,
+        fh::launch(dense_embedding_kernel<float>, dim3((ldx + 255) / 256, M), 256, 0, s, (const float*)table, width, scale, tokens_dev, x, ldx, next, (float*)out, ld_out,
                    (float*)out2, ld_out2, counts);
 }
 

@@ -356,6 +356,11 @@ int32_t forge_hip_attn_decode_sliding_f16kv(const float* q_dev, const uint16_t* 
                                             float* out_dev, uint32_t seq_len, uint32_t window, uint32_t heads,
                                             uint32_t kv_heads, uint32_t head_dim, uint32_t flags, void* stream);
 
+/* A dense product, y[M][N] = a[M][K] W[N][K]^T, as the networks of model folders compute it (matrix unit for M > 1, a
+ * matrix-vector kernel for M = 1): w_dev, a_dev row-major in `dtype` (FORGE_HIP_BF16 or FORGE_HIP_F32, full single precision),
+ * sums and y_dev in 32-bit.  K a multiple of 64, at most 32768; 16-byte aligned operands. */
+int32_t forge_hip_dense_matmul(uint32_t dtype, const void* w_dev, const void* a_dev, uint32_t M, uint32_t N, uint32_t K, float* y_dev, void* stream);
+
 /* argmax (project.rs:501-503): index of the LAST maximum of n floats -> *out_dev (uint32). */
 int32_t forge_hip_argmax(const float* x_dev, uint32_t n, uint32_t* out_dev, void* stream);
 
