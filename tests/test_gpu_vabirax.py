@@ -447,6 +447,16 @@ def test_other_number_formats_and_refusals(get, fh, vo, tmp_path):
         fh.HipModel.from_folder(str(tmp_path / "big"), 64)
 
 
+def test_command_line(get):
+    c = get("uneven")
+    root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+    prompt = c.ids(12, seed=62)
+    r = subprocess.run([sys.executable, os.path.join(root, "bin", "generate"), c.path, "--ids", ",".join(map(str, prompt)), "--max-tokens", "9",
+                        "--repeat-penalty", "1", "--dtype", "float32"], capture_output=True, text=True, timeout=100)
+    assert r.returncode == 0, r.stderr
+    assert [int(t) for t in r.stdout.split()[-1].split(",")] == c.oracle.greedy(prompt, 9)
+
+
 @pytest.mark.parametrize("dtype", DTYPES)
 def test_trace_replay(get, tmp_path, dtype):
     """bin/trace_run on a small trace: two requests, one after the other, prompt portions and single tokens."""
