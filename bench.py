@@ -471,7 +471,8 @@ def vabirax_bench(fh, args):
     if args.no_closest:
         print(js.dumps({"vabirax": line}))
         return
-    lcfg = getattr(fh.synth, "llama32_" + args.vabirax)(fh.Q8_0, max_seq=max_seq)
+    closest_name = {"135m": "smollm2_135m", "1b": "llama32_1b", "3b": "llama32_3b"}[args.vabirax]
+    lcfg = getattr(fh.synth, closest_name)(fh.Q8_0, max_seq=max_seq)
     blob = fh.synth.make_weights_blob(lcfg, seed=args.seed, threads=16)
     print("Llama weights made", file=sys.stderr, flush=True)
     gl = gemv_launch_bytes(fh, lcfg)
@@ -496,7 +497,7 @@ def vabirax_bench(fh, args):
                     "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
                     "config": {"model": "Vabirax " + args.vabirax, "prompt_tokens": n, "weights_bytes": nbytes, "write_s": round(t_write, 1),
                                "load_s": round(t_load, 1)},
-                    "vabirax": line, "closest_model": {"model": "Llama-3.2-%s shape, Q8_0" % args.vabirax.upper(), **closest}}))
+                    "vabirax": line, "closest_model": {"model": closest_name + " shape, Q8_0", **closest}}))
 
 
 def main():
@@ -522,7 +523,7 @@ def main():
     ap.add_argument("--ops-table", action="store_true",
                     help="instead of the model benchmark, run the isolated kernels at the benchmark configurations' sizes")
     ap.add_argument("--no-closest", action="store_true", help="with --vabirax: skip the Llama-family model")
-    ap.add_argument("--vabirax", choices=("1b", "3b"),
+    ap.add_argument("--vabirax", choices=("135m", "1b", "3b"),
                     help="instead of the default workload, the Vabirax design at this size beside the Llama-family model of the same size")
     args = ap.parse_args()
     if args.gpus != 1:

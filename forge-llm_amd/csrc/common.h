@@ -199,7 +199,7 @@ void launch_gemm(const QWeight& w, const int8_t* aq, const uint16_t* as, uint32_
                  bool accumulate, bool exact, int32_t* isums, hipStream_t s, void* split_ws = nullptr, int8_t* silu_q = nullptr,
                  uint16_t* silu_sc = nullptr, const float* mt_a = nullptr, const float* mt_w = nullptr);
 
-// model.hip — the part of forge_hip_model_create's checks that sizes depend on (formats, dimensions the kernels cover);
+// llama.hip — the part of forge_hip_model_create's checks that sizes depend on (formats, dimensions the kernels cover);
 // sets the error message.
 int32_t validate_config_shape(const forge_hip_config* c);
 

@@ -374,6 +374,12 @@ def vabirax_stream(config, seed) -> dict:
     return out
 
 
+def vabirax_135m() -> dict:
+    """SmolLM2-135M's width, depth and feed-forward; 9 heads of 64 + 32 (values 64), latents of 192 and 128, a window of 1024."""
+    layer = vabirax_layer(9, 64, 32, 64, 192, 128, 1536, 1024)
+    return vabirax_config(576, 49152, [layer] * 30, loop=(10, 20, 1), embedding_scale=24.0)
+
+
 def vabirax_1b() -> dict:
     """Layers of Llama-3.2-1B's width, depth and feed-forward; 16 heads of 128 + 64 (values 128), latents of 768 and 512."""
     layer = vabirax_layer(16, 128, 64, 128, 768, 512, 8192, 4096, base=500000.0)

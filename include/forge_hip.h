@@ -452,7 +452,9 @@ int32_t forge_hip_model_create_from_gguf(const char* path, uint32_t max_seq, uin
  * handle is an ordinary model: forward, forward_greedy, prefill, profile, repeat penalty and reset work as documented above
  * (forge_hip_model_set_kv_pages and forge_hip_model_read_kv: this network has a flat cache of latents, they are refused).
  * dtype: FORGE_HIP_BF16 (weights, activations and cache in bfloat16, 32-bit sums; norms, rotation, scores, softmax and the
- * residual stream in 32-bit) or FORGE_HIP_F32 (everything in 32-bit).  max_seq = 0: 4096 positions.  flags: 0. */
+ * residual stream in 32-bit) or FORGE_HIP_F32 (everything in 32-bit).  max_seq = 0: 4096 positions.  flags: 0.
+ * Limits: dim and rot_dim (each rounded up to 32) together at most 256, vdim at most 256, kv_rank at most 1024, width at most
+ * 16384, heads * vdim and ff at most 32768; every other size is free. */
 int32_t forge_hip_model_create_from_folder(const char* dir, uint32_t max_seq, uint32_t dtype, uint32_t flags, forge_hip_model** out);
 /* The sizes config.json gives, without a GPU (per-layer sizes: the first layer's; inter: the largest; max_seq and formats: 0). */
 int32_t forge_hip_folder_config(const char* dir, forge_hip_config* out);
