@@ -11,11 +11,13 @@ BUILD = os.path.join(HERE, "build")
 LIB = os.path.join(HERE, "libforge_hip.so")
 
 SOURCES = ["format.hip", "elementwise.hip", "gemv.hip", "gemv_f32.hip", "gemv_kquant.hip", "kquant_prefill.hip", "gemm.hip", "attn_decode.hip", "attn_prefill.hip",
-           "attn_exact.hip", "decode_persistent.hip", "api.hip", "model.hip", "llama.hip", "block_model.hip", "dense.hip", "attn_latent.hip", "checkpoint.cpp", "gguf.cpp", "sampling.cpp"]
+           "attn_exact.hip", "decode_persistent.hip", "api.hip", "model.hip", "llama.hip", "block_model.hip", "block_mixers.hip", "dense.hip",
+           "attn_prompt.hip", "attn_latent.hip", "attn_grouped.hip", "linear_attn.hip", "checkpoint.cpp", "gguf.cpp", "sampling.cpp"]
 
 # The trace replay program holds the dense networks only.
 TRACE_RUN = os.path.join(BUILD, "trace_run")
-TRACE_SOURCES = ["format.hip", "elementwise.hip", "model.hip", "block_model.hip", "dense.hip", "attn_latent.hip", "checkpoint.cpp", "trace_run.cpp"]
+TRACE_SOURCES = ["format.hip", "elementwise.hip", "model.hip", "block_model.hip", "block_mixers.hip", "dense.hip", "attn_prompt.hip", "attn_latent.hip", "attn_grouped.hip",
+                 "linear_attn.hip", "checkpoint.cpp", "trace_run.cpp"]
 
 # -packed-fp32-ops off: keep hipcc from forming packed FP32 instructions.
 # -ffp-contract=off: the CPU path never fuses a*b+c; kernels say fmaf() where a fused op is meant.

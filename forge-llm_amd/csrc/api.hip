@@ -461,7 +461,7 @@ int32_t forge_hip_dense_matmul(uint32_t dtype, const void* w_dev, const void* a_
     DenseEpiArgs e;
     e.f32 = y_dev;
     e.ld_f32 = N;
-    launch_dense((DType)dtype, w, a_dev, K, M, DenseEpi::F32, e, (hipStream_t)stream);
+    launch_dense((DType)dtype, w, dense_rows(a_dev, K), M, DenseEpi::F32, e, (hipStream_t)stream);
     FH_HIP(hipGetLastError());
     return FORGE_HIP_OK;
 }

@@ -302,6 +302,24 @@ struct Reader {
     }
 };
 
+// "rot": base, dims (even, at most `limit`) and, where the design has it, "scaling".
+void read_rotation(Reader& r, const Json& m, const std::string& at, uint32_t limit, bool scaling, RotarySpec* s) {
+    const Json* rot = r.object(m, "rot", at);
+    if (!rot) return;
+    const std::string in = at + "rot.";
+    s->dims = r.size(*rot, "dims", in);
+    s->base = r.number(*rot, "base", in);
+    if (!r.rc && (s->dims % 2 || s->dims > limit || s->base <= 0)) r.fail_at(at + "rot", "does not fit the head");
+    const Json* sc = scaling ? rot->get("scaling") : nullptr;
+    if (!sc || sc->kind == Json::Null) return;
+    if (sc->kind != Json::Object) { r.fail_at(in + "scaling", "must be an object"); return; }
+    s->factor = r.number(*sc, "factor", in + "scaling.");
+    s->low = r.number(*sc, "low", in + "scaling.");
+    s->high = r.number(*sc, "high", in + "scaling.");
+    s->original = r.number(*sc, "original", in + "scaling.");
+    if (!r.rc && (s->factor <= 0 || s->low <= 0 || s->high < s->low || s->original <= 0)) r.fail_at(in + "scaling", "makes no sense");
+}
+
 void read_latent_attention(Reader& r, const Json& m, const std::string& at, LatentAttentionSpec* s) {
     s->heads = r.size(m, "heads", at);
     s->dim = r.size(m, "dim", at);
@@ -310,11 +328,7 @@ void read_latent_attention(Reader& r, const Json& m, const std::string& at, Late
     s->q_rank = r.size(m, "q_rank", at);
     s->kv_rank = r.size(m, "kv_rank", at);
     s->scale = r.number(m, "scale", at);
-    if (const Json* rot = r.object(m, "rot", at)) {
-        s->rot.dims = r.size(*rot, "dims", at + "rot.");
-        s->rot.base = r.number(*rot, "base", at + "rot.");
-        if (!r.rc && (s->rot.dims % 2 || s->rot.dims > s->rot_dim || s->rot.base <= 0)) r.fail_at(at + "rot", "does not fit rot_dim");
-    }
+    read_rotation(r, m, at, s->rot_dim, false, &s->rot);
     const Json* mask = m.get("mask");
     if (mask && mask->kind != Json::Null) {
         const Json* size = mask->get("size");
@@ -323,31 +337,98 @@ void read_latent_attention(Reader& r, const Json& m, const std::string& at, Late
     }
 }
 
-// "Vabirax": looped decoder of latent-attention layers, Dynamic Tanh ahead of and behind every sublayer.
-int32_t parse_vabirax(const Json& c, BlockSpec* s) {
-    Reader r;
+void read_grouped_attention(Reader& r, const Json& m, const std::string& at, GroupedAttentionSpec* s) {
+    s->heads = r.size(m, "heads", at);
+    s->kv_heads = r.size(m, "kv_heads", at);
+    s->dim = r.size(m, "dim", at);
+    s->vdim = r.size(m, "vdim", at);
+    s->scale = r.number(m, "scale", at);
+    if (!r.rc && s->heads % s->kv_heads) r.fail_at(at + "kv_heads", "must divide heads");
+    read_rotation(r, m, at, s->dim, true, &s->rot);
+}
+
+void read_linear_attention(Reader& r, const Json& m, const std::string& at, LinearAttentionSpec* s) {
+    s->heads = r.size(m, "heads", at);
+    s->dim = r.size(m, "dim", at);
+    s->vdim = r.size(m, "vdim", at);
+    s->tau = r.number(m, "tau", at);
+    if (!r.rc && s->tau <= 0) r.fail_at(at + "tau", "must be positive");
+}
+
+// What every architecture's configuration starts with.
+void read_frame(Reader& r, const Json& c, BlockSpec* s) {
     s->width = r.size(c, "width", "");
     s->vocab = r.size(c, "vocab", "");
     if (const Json* e = r.object(c, "embedding", "")) s->embedding_scale = r.number(*e, "scale", "embedding.");
     if (const Json* n = r.object(c, "norm", "")) s->eps = r.number(*n, "eps", "norm.");
+}
+
+// "layers": a list of {type, mixer, mlp}; `mixer` reads a layer's mixer by its type and says whether it knows it.
+template <typename F>
+void read_layers(Reader& r, const Json& c, FeedForwardKind dense, BlockSpec* s, F mixer) {
     const Json* layers = c.get("layers");
-    if (!layers || layers->kind != Json::Array || layers->arr.empty()) { r.fail_at("layers", "must be a list"); return r.rc; }
+    if (!layers || layers->kind != Json::Array || layers->arr.empty()) { r.fail_at("layers", "must be a list"); return; }
     for (size_t i = 0; i < layers->arr.size() && !r.rc; i++) {
         const Json& l = layers->arr[i];
         const std::string at = "layers[" + std::to_string(i) + "].";
         LayerSpec ls;
+        ls.weights = (uint32_t)i;
         const Json* type = l.get("type");
-        if (!type || type->kind != Json::String || type->str != "latent_attention") { r.fail_at(at + "type", "must be \"latent_attention\""); break; }
-        if (const Json* m = r.object(l, "mixer", at)) read_latent_attention(r, *m, at + "mixer.", &ls.latent);
+        if (!type || type->kind != Json::String) { r.fail_at(at + "type", "must be a string"); break; }
+        const Json* m = r.object(l, "mixer", at);
+        if (!m) break;
+        if (!mixer(type->str, *m, at + "mixer.", &ls)) { r.fail_at(at + "type", "is no mixer of this architecture"); break; }
         const Json* mlp = l.get("mlp");
         if (mlp && mlp->kind != Json::Null) {
             const Json* kind = mlp->get("kind");
             if (!kind || kind->kind != Json::String || kind->str != "dense") { r.fail_at(at + "mlp.kind", "must be \"dense\""); break; }
-            ls.ff = FeedForwardKind::SiluGated;
+            ls.ff = dense;
             ls.ff_size = r.size(*mlp, "ff", at + "mlp.");
         }
         s->layers.push_back(ls);
     }
+}
+
+// "weights_of": j in a layer's entry: the layer runs with layer j's tensors, and the rest of its entry equals j's.
+void read_shared_weights(Reader& r, const Json& c, BlockSpec* s) {
+    auto same = [](const LayerSpec& a, const LayerSpec& b) {
+        auto rot = [](const RotarySpec& x, const RotarySpec& y) { return !(x < y) && !(y < x); };
+        const GroupedAttentionSpec &g = a.grouped, &h = b.grouped;
+        const LinearAttentionSpec &l = a.linear, &m = b.linear;
+        return a.mixer == b.mixer && a.ff == b.ff && a.ff_size == b.ff_size && g.heads == h.heads && g.kv_heads == h.kv_heads && g.dim == h.dim &&
+               g.vdim == h.vdim && g.scale == h.scale && rot(g.rot, h.rot) && l.heads == m.heads && l.dim == m.dim && l.vdim == m.vdim && l.tau == m.tau;
+    };
+    const size_t n = s->layers.size();
+    for (size_t i = 0; i < n && !r.rc; i++) {
+        const Json& l = c.get("layers")->arr[i];
+        const std::string at = "layers[" + std::to_string(i) + "].";
+        const Json* of = l.get("weights_of");
+        if (!of || of->kind == Json::Null) continue;
+        s->layers[i].weights = r.size(l, "weights_of", at, 0);
+        if (!r.rc && s->layers[i].weights >= n) r.fail_at(at + "weights_of", "names no layer");
+    }
+    // a layer named may itself borrow: follow to the one that has tensors
+    for (size_t i = 0; i < n && !r.rc; i++) {
+        uint32_t j = s->layers[i].weights;
+        for (size_t hops = 0; j != s->layers[j].weights && hops <= n; hops++) j = s->layers[j].weights;
+        const std::string at = "layers[" + std::to_string(i) + "].weights_of";
+        if (j != s->layers[j].weights) r.fail_at(at, "goes round in a circle");
+        else if (!same(s->layers[i], s->layers[j])) r.fail_at(at, "names a layer of another shape");
+        s->layers[i].weights = j;
+    }
+}
+
+// "Vabirax": looped decoder of latent-attention layers, Dynamic Tanh ahead of and behind every sublayer.
+int32_t parse_vabirax(const Json& c, BlockSpec* s) {
+    Reader r;
+    s->post_norms = true;
+    read_frame(r, c, s);
+    read_layers(r, c, FeedForwardKind::SiluGated, s, [&](const std::string& type, const Json& m, const std::string& at, LayerSpec* l) {
+        if (type != "latent_attention") return false;
+        l->mixer = MixerKind::LatentAttention;
+        read_latent_attention(r, m, at, &l->latent);
+        return true;
+    });
     const Json* loop = c.get("loop");
     if (loop && loop->kind != Json::Null && !r.rc) {
         s->loop_start = r.size(*loop, "start", "loop.", 0);
@@ -358,15 +439,54 @@ int32_t parse_vabirax(const Json& c, BlockSpec* s) {
     return r.rc;
 }
 
+// "Kakirax": decoder that mixes gated linear attention and grouped-query attention layers, a layer norm ahead of every sublayer;
+// layers may share weights, the output matrix is the embedding table, logits are capped.
+int32_t parse_kakirax(const Json& c, BlockSpec* s) {
+    Reader r;
+    s->norm = NormKind::LayerNorm;
+    s->tied_head = true;
+    read_frame(r, c, s);
+    const Json* cap = c.get("logit_softcap");
+    if (cap && cap->kind != Json::Null) {
+        s->logit_cap = r.number(c, "logit_softcap", "");
+        if (!r.rc && s->logit_cap <= 0) r.fail_at("logit_softcap", "must be positive");
+    }
+    read_layers(r, c, FeedForwardKind::GeluTanhGated, s, [&](const std::string& type, const Json& m, const std::string& at, LayerSpec* l) {
+        if (type == "attention") {
+            l->mixer = MixerKind::GroupedAttention;
+            read_grouped_attention(r, m, at, &l->grouped);
+        } else if (type == "gla") {
+            l->mixer = MixerKind::LinearAttention;
+            read_linear_attention(r, m, at, &l->linear);
+        } else {
+            return false;
+        }
+        return true;
+    });
+    if (!r.rc) read_shared_weights(r, c, s);
+    return r.rc;
+}
+
 struct Architecture {
     const char* name;
     int32_t (*parse)(const Json& config, BlockSpec* out);
 };
 const Architecture ARCHITECTURES[] = {
     {"Vabirax", parse_vabirax},
+    {"Kakirax", parse_kakirax},
 };
 
 }  // namespace
+
+double RotarySpec::frequency(uint32_t i) const {
+    const double f = pow(base, -2.0 * i / dims);
+    if (factor == 0) return f;
+    const double length = 2 * M_PI / f;
+    if (length < original / high) return f;
+    if (length > original / low) return f / factor;
+    const double s = high > low ? (original / length - low) / (high - low) : 1.0;
+    return (1 - s) * f / factor + s * f;
+}
 
 bool architecture_known(const std::string& architecture) {
     for (const Architecture& a : ARCHITECTURES)

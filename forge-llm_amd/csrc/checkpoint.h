@@ -7,6 +7,7 @@
 #include <map>
 #include <memory>
 #include <string>
+#include <tuple>
 #include <vector>
 
 namespace fh {
@@ -61,8 +62,15 @@ private:
 
 // ---- network description -------------------------------------------------------------------------
 struct RotarySpec {
-    uint32_t dims = 0;                   // dimension i turns against i + dims / 2 by position * base^(-2 i / dims)
+    uint32_t dims = 0;                   // dimension i turns against i + dims / 2 by position * frequency(i)
     double base = 0;
+    // Stretched frequencies: waves longer than original / low turn `factor` times slower, those shorter than original / high as they
+    // are, with a blend between.  factor = 0: none.
+    double factor = 0, low = 0, high = 0, original = 0;
+    double frequency(uint32_t i) const;  // base^(-2 i / dims), stretched
+    bool operator<(const RotarySpec& o) const {
+        return std::tie(dims, base, factor, low, high, original) < std::tie(o.dims, o.base, o.factor, o.low, o.high, o.original);
+    }
 };
 struct LatentAttentionSpec {
     uint32_t heads = 0, dim = 0, rot_dim = 0, vdim = 0, q_rank = 0, kv_rank = 0;
@@ -70,18 +78,37 @@ struct LatentAttentionSpec {
     double scale = 0;
     RotarySpec rot;
 };
-enum class MixerKind { LatentAttention };
-enum class FeedForwardKind { None, SiluGated };
+// Grouped-query attention: queries and keys normed per head (RMS) and rotated, a sigmoid gate on the heads' output.
+struct GroupedAttentionSpec {
+    uint32_t heads = 0, kv_heads = 0, dim = 0, vdim = 0;
+    double scale = 0;
+    RotarySpec rot;
+};
+// Gated linear attention: a decay per key channel, sigmoid(low-rank map)^(1 / tau); the map's rank is its tensors'.
+struct LinearAttentionSpec {
+    uint32_t heads = 0, dim = 0, vdim = 0;
+    double tau = 0;
+};
+enum class MixerKind { LatentAttention, GroupedAttention, LinearAttention };
+enum class FeedForwardKind { None, SiluGated, GeluTanhGated };
+enum class NormKind { DynTanh, LayerNorm };
 struct LayerSpec {
     MixerKind mixer = MixerKind::LatentAttention;
     LatentAttentionSpec latent;
+    GroupedAttentionSpec grouped;
+    LinearAttentionSpec linear;
     FeedForwardKind ff = FeedForwardKind::None;
     uint32_t ff_size = 0;
+    uint32_t weights = 0;                // the layer whose tensors this one runs with (its own index, or another's)
 };
 struct BlockSpec {
     std::string architecture;
     uint32_t width = 0, vocab = 0;
     double embedding_scale = 1, eps = 0;
+    NormKind norm = NormKind::DynTanh;
+    bool post_norms = false;             // a norm behind each sublayer, ahead of the residual sum
+    bool tied_head = false;              // the embedding table is the output matrix
+    double logit_cap = 0;                // logits <- cap tanh(logits / cap); 0: as they are
     std::vector<LayerSpec> layers;
     // layers [loop_start, loop_stop) run loop_times times in a row with the same weights and a cache per pass; ahead of each
     // pass x <- W [x; embedding output].  loop_times = 0: no loop.

@@ -266,14 +266,22 @@ struct DynTanh {
     const float* b = nullptr;
     float alpha = 0.f;
 };
+// (x - mean) / sqrt(variance + eps) * w + b over the first `n` elements of a row; w and b are zero past them.
+struct LayerNorm {
+    const float* w = nullptr;
+    const float* b = nullptr;
+    uint32_t n = 0;
+    float eps = 0.f;
+};
+enum class Act : uint32_t { Sigmoid, Silu, GeluTanh };
 enum class DenseEpi {
-    F32,        // f32[m][n] = v
-    RawGate,    // columns below `split`: f32[m][n] = v; the others: out[m][n - split] = sigmoid(v)
+    F32,        // f32[m][n] = v, or cap * tanh(v / cap) with a cap
+    RawGate,    // columns below `split`: f32[m][n] = v; the others: out[m][n - split] = act(v)
     Rope,       // heads of head_stride columns: the pairs (rot_off + 2 i, rot_off + 2 i + 1), i < rot_pairs, turn by the angle of (position, i); out = the result
     Split,      // columns below `split` go to out, the others to out2
     GateMul,    // out = v * gate
-    SiluPair,   // columns 2 i and 2 i + 1 are gate and up: out[m][i] = silu(gate) * up
-    Residual,   // a = post(v) (+ f32 if add); f32 = a; out = next(a)
+    ActPair,    // columns 2 i and 2 i + 1 are gate and up: out[m][i] = act(gate) * up
+    Residual,   // a = post(v) (+ f32 if add); f32 = a; out (optional) = next(a)
 };
 struct DenseEpiArgs {
     float* f32 = nullptr;
@@ -283,6 +291,8 @@ struct DenseEpiArgs {
     void* out2 = nullptr;
     uint32_t ld_out2 = 0;
     uint32_t split = 0;
+    Act act = Act::Sigmoid;
+    float cap = 0.f;
     const void* gate = nullptr;      // [m][ld_out]
     DynTanh post, next;
     int add = 0;
@@ -292,14 +302,110 @@ struct DenseEpiArgs {
     const uint32_t* pos_dev = nullptr;
     uint32_t head_stride = 1, rot_off = 0, rot_pairs = 0;
 };
+// What a product multiplies: stored rows, or (one row only) something its kernel makes from 32-bit values on the way in.
+struct DenseIn {
+    enum Kind : uint32_t {
+        Rows,       // rows of `lda` elements
+        Normed,     // layer norm of `f32` (RawGate and ActPair)
+        HeadGate,   // per head of `head` columns: RMS norm of `f32` over the first head_n of them, * w, * gate (Residual)
+    } kind = Rows;
+    const void* rows = nullptr;
+    uint32_t lda = 0;
+    const float* f32 = nullptr;
+    LayerNorm ln;
+    uint32_t heads = 0, head = 0, head_n = 0;
+    const float* w = nullptr;        // [head]
+    const void* gate = nullptr;      // [heads * head]
+    float eps = 0.f;
+};
+inline DenseIn dense_rows(const void* rows, uint32_t lda) { DenseIn in; in.rows = rows; in.lda = lda; return in; }
 // y = a W^T over M rows, then the epilogue.  One row runs as a matrix-vector kernel.
-void launch_dense(DType t, const DenseWeight& w, const void* a, uint32_t lda, uint32_t M, DenseEpi mode, const DenseEpiArgs& e, hipStream_t s);
+void launch_dense(DType t, const DenseWeight& w, const DenseIn& in, uint32_t M, DenseEpi mode, const DenseEpiArgs& e, hipStream_t s);
 uint32_t dense_k_max();
-// x[m] = table[token[m]] * scale (f32, rows of ldx, zero past `width`), out = next(x), out2 (optional) = x; counts as in launch_embedding.
-void launch_dense_embedding(DType t, const void* table, uint32_t width, float scale, const uint32_t* tokens_dev, uint32_t M, float* x,
+// out[m] = layer norm of x[m]; rows of `width` elements (a multiple of 64, at most 16384), those past ln.n come out zero
+void launch_layer_norm(DType t, const float* x, uint32_t ldx, const LayerNorm& ln, uint32_t width, uint32_t M, void* out, uint32_t ld_out, hipStream_t s);
+// x[m] = table[token[m]] * scale (f32, rows of ldx, zero past `width`), out (optional) = next(x), out2 (optional) = x; the table's rows
+// are `ld_table` elements apart; counts as in launch_embedding.
+void launch_dense_embedding(DType t, const void* table, uint32_t ld_table, uint32_t width, float scale, const uint32_t* tokens_dev, uint32_t M, float* x,
                             uint32_t ldx, const DynTanh& next, void* out, uint32_t ld_out, void* out2, uint32_t ld_out2, uint32_t* counts, hipStream_t s);
 // out[i] = a[rows[i]] for n rows of `width` elements
 void launch_gather_rows(DType t, const void* a, uint32_t lda, const uint32_t* rows_dev, uint32_t n, uint32_t width, void* out, uint32_t ld_out, hipStream_t s);
+
+// attn_prompt.hip — causal attention of a prompt's rows over dense keys and values, softmax(scale q k^T) v * gate.  A key is `dim`
+// columns of its head in `k` and, behind them, `rot` columns that all heads share (`shared`, may be absent).  Sizes are multiples of 32.
+struct PromptAttn {
+    uint32_t heads = 0, group = 1;           // `group` query heads in a row share a key / value head
+    uint32_t dim = 0, rot = 0, vdim = 0;
+    uint32_t window = 0;                     // a row sees itself and the window - 1 positions before it; 0: every earlier position
+    float scale = 0.f;
+    const void* q = nullptr;                 // [M][heads][dim + rot]
+    const void* k = nullptr;                 // rows of k_row elements from position kv_lo (a multiple of 64) on
+    const void* v = nullptr;                 // rows of v_row elements, likewise
+    const void* shared = nullptr;            // rows of shared_row elements from position 0 on
+    uint32_t k_row = 0, v_row = 0, shared_row = 0, kv_lo = 0;
+    const void* gate = nullptr;              // [M][ld_out]
+    void* out = nullptr;
+    uint32_t ld_out = 0;
+};
+constexpr uint32_t DENSE_HEAD_MAX = 256;     // dim + rot, vdim
+void launch_attn_prompt(DType t, const PromptAttn& a, uint32_t M, uint32_t base_pos, hipStream_t s);
+
+// attn_grouped.hip — grouped-query attention with an RMS norm and a rotation per query and key head, over a flat cache of K rows
+// [kv_heads][dim] and V rows [kv_heads][vdim].  Sizes are the padded ones of the buffers (multiples of 32); rotary partners lie side by side.
+struct GroupedShape {
+    uint32_t heads = 0, kv_heads = 0, dim = 0, vdim = 0;
+    uint32_t dim_n = 0;                      // elements a head's norm counts
+    uint32_t rot_pairs = 0;
+    float scale = 0.f, eps = 0.f;
+    __host__ __device__ uint32_t group() const { return heads / kv_heads; }
+    __host__ __device__ uint32_t k_row() const { return kv_heads * dim; }
+    __host__ __device__ uint32_t v_row() const { return kv_heads * vdim; }
+    __host__ __device__ uint32_t raw_row() const { return heads * dim + k_row() + v_row(); }
+};
+struct GroupedIo {
+    const float* raw;                        // [M][q | k | v] of the positions at hand
+    const float* q_norm;                     // [dim]
+    const float* k_norm;
+    const float* cos_t;
+    const float* sin_t;
+    void* k_cache;                           // [max_seq][kv_heads][dim]
+    void* v_cache;
+    uint32_t max_seq, base_pos;
+    const uint32_t* pos_dev;                 // one row only
+};
+// Prompt rows: q [M][heads][dim] = rotated norm of the raw queries; cache rows base_pos.. = rotated norm of the raw keys, raw values
+void launch_grouped_norm_store(DType t, const GroupedShape& sh, const GroupedIo& io, uint32_t M, void* q, hipStream_t s);
+// One row, two launches: the new cache row and attention in up to grouped_splits() parts, then [merge of the parts | gate] -> out.
+uint32_t grouped_splits(const GroupedShape& sh, uint32_t max_seq);
+size_t grouped_parts_bytes(const GroupedShape& sh, uint32_t max_seq);
+void launch_grouped_decode(DType t, const GroupedShape& sh, const GroupedIo& io, float* parts, const void* gate, void* out, hipStream_t s);
+
+// linear_attn.hip — gated linear attention: per head a matrix S [dim][vdim] in 32-bit, S <- diag(a) S + k v^T, o = S^T q, with a decay
+// per key channel a = sigmoid(W2 low + b)^(1 / tau).  All of it in 32-bit for both element types.  Padded sizes (multiples of 32).
+struct LinearShape {
+    uint32_t heads = 0, dim = 0, vdim = 0;
+    uint32_t rank = 0;                       // of the decay's low-rank map (a multiple of 4)
+    uint32_t vdim_n = 0;                     // elements a head's output norm counts
+    float q_scale = 0.f, inv_tau = 0.f, eps = 0.f;
+    __host__ __device__ uint32_t qk() const { return heads * dim; }
+    __host__ __device__ uint32_t raw_row() const { return 2 * qk() + heads * vdim + rank; }
+    __host__ __device__ size_t state() const { return (size_t)heads * dim * vdim; }
+};
+struct LinearIo {
+    const float* raw;                        // [M][q | k | v | low]
+    const float* w2;                         // [rank][heads * dim]
+    const float* b2;                         // [heads * dim]
+    float* state;                            // [heads][dim][vdim]; what it holds at position 0 is not looked at
+    uint32_t base_pos;
+    const uint32_t* pos_dev;                 // one row only
+};
+bool linear_shape_supported(const LinearShape& sh);
+// Prompt rows in chunks of 64: out [M][ld_out] = RMS norm of o per head * norm * gate.  work: linear_work_bytes(sh, M).
+size_t linear_work_bytes(const LinearShape& sh, uint32_t M);
+void launch_linear_prompt(DType t, const LinearShape& sh, const LinearIo& io, uint32_t M, float* work, const float* norm, const void* gate, void* out,
+                          uint32_t ld_out, hipStream_t s);
+// One row: state and o [heads][vdim] (norm and gate are the output product's, DenseIn::HeadGate).
+void launch_linear_step(const LinearShape& sh, const LinearIo& io, float* o, hipStream_t s);
 
 // attn_latent.hip — attention whose keys and values are linear maps of one cached latent vector per position, beside one rotated
 // key part that all heads share.  Sizes are the padded ones of the buffers (multiples of 32; the latent a multiple of 64).
@@ -317,10 +423,6 @@ bool latent_shape_supported(DType t, const LatentShape& sh);
 // raw f32 [M][q_rank | rank | rot] -> cq [M][q_rank] = RMSnorm * q_norm; cache row of the position = RMSnorm * kv_norm | rotated part
 void launch_latent_norm_store(DType t, const LatentShape& sh, const float* raw, const float* q_norm, const float* kv_norm, const float* cos_t,
                               const float* sin_t, uint32_t M, uint32_t base_pos, void* cq, void* cache, hipStream_t s);
-// Prompt form: keys and values expanded per head, kbuf [positions kv_lo..][heads][dim], vbuf [..][heads][vdim] (kv_lo a multiple of
-// 64), the rotated key part from the cache; out [M][ld_out] = attention * gate.
-void launch_latent_attn_prefill(DType t, const LatentShape& sh, const void* q, const void* kbuf, const void* vbuf, const void* cache, uint32_t kv_lo,
-                                const void* gate, void* out, uint32_t ld_out, uint32_t M, uint32_t base_pos, hipStream_t s);
 // One row at pos_dev ? *pos_dev : base_pos, four launches: [norm of the query latent | W_uq | rotation] beside the new cache row,
 // queries taken to the latent space (W_uk^T q per head), attention over the cached latents in up to latent_splits() parts, and
 // [merge of the parts | W_uv | gate].

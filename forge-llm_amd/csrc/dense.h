@@ -71,6 +71,20 @@ __device__ __forceinline__ v4f mma16(v8f a, v8f b, v4f c) {
 __device__ __forceinline__ float dyn_tanh(const DynTanh& t, uint32_t n, float x) { return t.w ? tanhf(t.alpha * x) * t.w[n] + t.b[n] : x; }
 __device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float silu_f(float z) { return z / (1.0f + expf(-z)); }
+// 0.5 z (1 + tanh(u)) with u = sqrt(2 / pi) (z + 0.044715 z^3): the logistic function of 2 u, times z
+__device__ __forceinline__ float gelu_tanh_f(float z) { return z / (1.0f + expf(-1.5957691216057308f * (z + 0.044715f * z * z * z))); }
+__device__ __forceinline__ float act_f(Act a, float z) { return a == Act::Sigmoid ? sigmoid_f(z) : a == Act::Silu ? silu_f(z) : gelu_tanh_f(z); }
+
+// Sum over the workgroup of `nt` threads; red: LDS, nt / 64 floats, free again after the next barrier.
+__device__ __forceinline__ float block_sum(float v, float* red, uint32_t tid, uint32_t nt) {
+    v = wave_sum(v);
+    __syncthreads();
+    if ((tid & 63) == 0) red[tid >> 6] = v;
+    __syncthreads();
+    float s = 0.f;
+    for (uint32_t i = 0; i < nt / 64; i++) s += red[i];
+    return s;
+}
 
 // What happens to the results (m, n .. n + 3) of a product; n is a multiple of 4.
 template <typename T, DenseEpi MODE>
@@ -79,10 +93,10 @@ __device__ __forceinline__ void dense_epilogue(const DenseEpiArgs& e, uint32_t m
         float* y = e.f32 + (size_t)m * e.ld_f32 + n;
 #pragma unroll
         for (int i = 0; i < 4; i++)
-            if (n + i < N) y[i] = v[i];
+            if (n + i < N) y[i] = e.cap > 0.f ? e.cap * tanhf(v[i] / e.cap) : v[i];
     } else if constexpr (MODE == DenseEpi::RawGate) {
         if (n < e.split) *reinterpret_cast<float4*>(e.f32 + (size_t)m * e.ld_f32 + n) = make_float4(v[0], v[1], v[2], v[3]);
-        else store4<T>((T*)e.out + (size_t)m * e.ld_out + (n - e.split), sigmoid_f(v[0]), sigmoid_f(v[1]), sigmoid_f(v[2]), sigmoid_f(v[3]));
+        else store4<T>((T*)e.out + (size_t)m * e.ld_out + (n - e.split), act_f(e.act, v[0]), act_f(e.act, v[1]), act_f(e.act, v[2]), act_f(e.act, v[3]));
     } else if constexpr (MODE == DenseEpi::Rope) {
         const uint32_t j = n % e.head_stride;
         float a[4] = {v[0], v[1], v[2], v[3]};
@@ -106,10 +120,10 @@ __device__ __forceinline__ void dense_epilogue(const DenseEpiArgs& e, uint32_t m
     } else if constexpr (MODE == DenseEpi::GateMul) {
         const T* g = (const T*)e.gate + (size_t)m * e.ld_out + n;
         store4<T>((T*)e.out + (size_t)m * e.ld_out + n, v[0] * (float)g[0], v[1] * (float)g[1], v[2] * (float)g[2], v[3] * (float)g[3]);
-    } else if constexpr (MODE == DenseEpi::SiluPair) {
+    } else if constexpr (MODE == DenseEpi::ActPair) {
         T* y = (T*)e.out + (size_t)m * e.ld_out + n / 2;
-        y[0] = (T)(silu_f(v[0]) * v[1]);
-        y[1] = (T)(silu_f(v[2]) * v[3]);
+        y[0] = (T)(act_f(e.act, v[0]) * v[1]);
+        y[1] = (T)(act_f(e.act, v[2]) * v[3]);
     } else if constexpr (MODE == DenseEpi::Residual) {
         // everything the four results need is requested at once
         float4* xp = reinterpret_cast<float4*>(e.f32 + (size_t)m * e.ld_f32 + n);
@@ -128,6 +142,7 @@ __device__ __forceinline__ void dense_epilogue(const DenseEpiArgs& e, uint32_t m
         norm4(e.post, pw, pb);
         a[0] += x.x; a[1] += x.y; a[2] += x.z; a[3] += x.w;
         *xp = make_float4(a[0], a[1], a[2], a[3]);
+        if (!e.out) return;
         norm4(e.next, nw, nb);
         store4<T>((T*)e.out + (size_t)m * e.ld_out + n, a[0], a[1], a[2], a[3]);
     }

@@ -116,28 +116,112 @@ void dense_gemm_kernel(const T* __restrict__ w, const T* __restrict__ a, uint32_
     }
 }
 
-template <typename T, int KS, DenseEpi MODE>
-__global__ __launch_bounds__(GEMV_THREADS) void dense_gemv_kernel(const T* __restrict__ w, const T* __restrict__ a, uint32_t N, uint32_t K, DenseEpiArgs e) {
+// The vector of a one-row product goes into LDS as floats, made from what DenseIn names.
+template <typename T, int KS, DenseEpi MODE, DenseIn::Kind IN>
+__global__ __launch_bounds__(GEMV_THREADS) void dense_gemv_kernel(const T* __restrict__ w, DenseIn in, uint32_t N, uint32_t K, DenseEpiArgs e) {
     extern __shared__ __attribute__((aligned(16))) float gemv_lds[];
+    const uint32_t tid = threadIdx.x;
     float* xs = gemv_lds;
-    gemv_body<T, KS, MODE>(w, N, K, blockIdx.x * gemv_rows<KS>(), xs, gemv_lds + K, e, [&]() {
-        for (uint32_t k = threadIdx.x * 8; k < K; k += GEMV_THREADS * 8) {
-            const typename Vec<T>::x8 v = load8(a + k);
+    float* red = gemv_lds + K;
+    gemv_body<T, KS, MODE>(w, N, K, blockIdx.x * gemv_rows<KS>(), xs, red, e, [&]() {
+        if constexpr (IN == DenseIn::Rows) {
+            const T* a = (const T*)in.rows;
+            for (uint32_t k = tid * 8; k < K; k += GEMV_THREADS * 8) {
+                const typename Vec<T>::x8 v = load8(a + k);
 #pragma unroll
-            for (int j = 0; j < 8; j++) xs[k + j] = (float)v[j];
+                for (int j = 0; j < 8; j++) xs[k + j] = (float)v[j];
+            }
+        } else if constexpr (IN == DenseIn::Normed) {
+            // a thread keeps to its own elements until the product's barrier
+            float s = 0.f;
+            for (uint32_t k = tid * 4; k < K; k += GEMV_THREADS * 4) {
+                const v4f v = *reinterpret_cast<const v4f*>(in.f32 + k);
+                *reinterpret_cast<v4f*>(xs + k) = v;
+                s += (v[0] + v[1]) + (v[2] + v[3]);                       // zero past ln.n
+            }
+            const float mean = block_sum(s, red, tid, GEMV_THREADS) / (float)in.ln.n;
+            float ss = 0.f;
+            for (uint32_t k = tid * 4; k < K; k += GEMV_THREADS * 4)
+#pragma unroll
+                for (int j = 0; j < 4; j++) {
+                    const float d = xs[k + j] - mean;
+                    if (k + j < in.ln.n) ss = fmaf(d, d, ss);
+                }
+            const float inv = 1.0f / sqrtf(block_sum(ss, red, tid, GEMV_THREADS) / (float)in.ln.n + in.ln.eps);
+            for (uint32_t k = tid * 4; k < K; k += GEMV_THREADS * 4) {
+                const v4f lw = *reinterpret_cast<const v4f*>(in.ln.w + k), lb = *reinterpret_cast<const v4f*>(in.ln.b + k);
+#pragma unroll
+                for (int j = 0; j < 4; j++) xs[k + j] = (xs[k + j] - mean) * inv * lw[j] + lb[j];
+            }
+        } else {
+            // head = a multiple of 32 columns: lane group of 16, 4 columns per lane and step
+            const uint32_t n = in.heads * in.head;
+            for (uint32_t k = n + tid; k < K; k += GEMV_THREADS) xs[k] = 0.f;
+            for (uint32_t h = tid / 16; h < in.heads; h += GEMV_THREADS / 16) {
+                const float* o = in.f32 + h * in.head;
+                float ss = 0.f;
+                for (uint32_t c = tid % 16 * 4; c < in.head; c += 64) {
+                    const v4f v = *reinterpret_cast<const v4f*>(o + c);
+#pragma unroll
+                    for (int j = 0; j < 4; j++) ss = fmaf(v[j], v[j], ss);      // zero past head_n
+                }
+                ss = lane_xor_add<8>(ss); ss = lane_xor_add<4>(ss); ss = lane_xor_add<2>(ss); ss = lane_xor_add<1>(ss);
+                const float inv = 1.0f / sqrtf(ss / (float)in.head_n + in.eps);
+                for (uint32_t c = tid % 16 * 4; c < in.head; c += 64) {
+                    const v4f v = *reinterpret_cast<const v4f*>(o + c), hw = *reinterpret_cast<const v4f*>(in.w + c);
+                    const typename Vec<T>::x4 g = *reinterpret_cast<const typename Vec<T>::x4*>((const T*)in.gate + h * in.head + c);
+#pragma unroll
+                    for (int j = 0; j < 4; j++) xs[h * in.head + c + j] = v[j] * inv * hw[j] * (float)g[j];
+                }
+            }
         }
     });
 }
 
+// One workgroup per row; a thread holds NV groups of four elements.
+template <typename T, int NV>
+__global__ __launch_bounds__(256) void layer_norm_kernel(const float* __restrict__ x, uint32_t ldx, LayerNorm ln, uint32_t width, T* __restrict__ out, uint32_t ld_out) {
+    __shared__ float red[4];
+    const uint32_t m = blockIdx.x, tid = threadIdx.x;
+    v4f v[NV];
+    float s = 0.f;
+#pragma unroll
+    for (int i = 0; i < NV; i++) {
+        const uint32_t c = (tid + 256 * i) * 4;
+        v[i] = c < width ? *reinterpret_cast<const v4f*>(x + (size_t)m * ldx + c) : (v4f){0.f, 0.f, 0.f, 0.f};
+        s += (v[i][0] + v[i][1]) + (v[i][2] + v[i][3]);                  // zero past ln.n
+    }
+    const float mean = block_sum(s, red, tid, 256) / (float)ln.n;
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < NV; i++)
+#pragma unroll
+        for (int j = 0; j < 4; j++) {
+            const float d = v[i][j] - mean;
+            if ((tid + 256 * i) * 4 + j < ln.n) ss = fmaf(d, d, ss);
+        }
+    const float inv = 1.0f / sqrtf(block_sum(ss, red, tid, 256) / (float)ln.n + ln.eps);
+#pragma unroll
+    for (int i = 0; i < NV; i++) {
+        const uint32_t c = (tid + 256 * i) * 4;
+        if (c >= width) continue;
+        const v4f w = *reinterpret_cast<const v4f*>(ln.w + c), b = *reinterpret_cast<const v4f*>(ln.b + c);
+        float y[4];
+#pragma unroll
+        for (int j = 0; j < 4; j++) y[j] = (v[i][j] - mean) * inv * w[j] + b[j];
+        store4<T>(out + (size_t)m * ld_out + c, y[0], y[1], y[2], y[3]);
+    }
+}
+
 template <typename T>
-__global__ __launch_bounds__(256) void dense_embedding_kernel(const T* __restrict__ table, uint32_t width, float scale, const uint32_t* __restrict__ tokens,
+__global__ __launch_bounds__(256) void dense_embedding_kernel(const T* __restrict__ table, uint32_t ld_table, uint32_t width, float scale, const uint32_t* __restrict__ tokens,
                                                               float* __restrict__ x, uint32_t ldx, DynTanh next, T* __restrict__ out, uint32_t ld_out,
                                                               T* __restrict__ out2, uint32_t ld_out2, uint32_t* __restrict__ counts) {
     const uint32_t m = blockIdx.y, tok = tokens[m], i = blockIdx.x * 256 + threadIdx.x;
     if (i < ldx) {
-        const float v = i < width ? (float)table[(size_t)tok * width + i] * scale : 0.f;
+        const float v = i < width ? (float)table[(size_t)tok * ld_table + i] * scale : 0.f;
         x[(size_t)m * ldx + i] = v;
-        out[(size_t)m * ld_out + i] = (T)dyn_tanh(next, i, v);
+        if (out) out[(size_t)m * ld_out + i] = (T)dyn_tanh(next, i, v);
         if (out2) out2[(size_t)m * ld_out2 + i] = (T)v;
     }
     if (i == 0 && counts) atomicAdd(counts + tok, 1u);
@@ -161,25 +245,34 @@ void go_gemm(const DenseWeight& w, const void* a, uint32_t lda, uint32_t M, cons
     fh::launch(dense_gemm_kernel<T, TN, TM, MODE>, dim3(tn * tm), 256, lds, s, (const T*)w.p, (const T*)a, lda, M, w.N, w.K, tn, e);
 }
 
-template <typename T, int KS, DenseEpi MODE>
-void go_gemv(const DenseWeight& w, const void* a, const DenseEpiArgs& e, hipStream_t s) {
-    static const hipError_t lds_ok = hipFuncSetAttribute((const void*)dense_gemv_kernel<T, KS, MODE>, hipFuncAttributeMaxDynamicSharedMemorySize, (DENSE_K_MAX + 16) * 4);
+template <typename T, int KS, DenseEpi MODE, DenseIn::Kind IN>
+void go_gemv(const DenseWeight& w, const DenseIn& in, const DenseEpiArgs& e, hipStream_t s) {
+    static const hipError_t lds_ok = hipFuncSetAttribute((const void*)dense_gemv_kernel<T, KS, MODE, IN>, hipFuncAttributeMaxDynamicSharedMemorySize, (DENSE_K_MAX + 16) * 4);
     (void)lds_ok;
-    fh::launch(dense_gemv_kernel<T, KS, MODE>, dim3((w.N + gemv_rows<KS>() - 1) / gemv_rows<KS>()), GEMV_THREADS, (w.K + 16) * 4, s, (const T*)w.p,
-               (const T*)a, w.N, w.K, e);
+    fh::launch(dense_gemv_kernel<T, KS, MODE, IN>, dim3((w.N + gemv_rows<KS>() - 1) / gemv_rows<KS>()), GEMV_THREADS, (w.K + 16) * 4, s, (const T*)w.p,
+               in, w.N, w.K, e);
+}
+
+template <typename T, DenseEpi MODE, DenseIn::Kind IN>
+void go_row(const DenseWeight& w, const DenseIn& in, const DenseEpiArgs& e, hipStream_t s) {
+    switch (gemv_depth_split(w.N, w.K)) {
+        case 1: go_gemv<T, 1, MODE, IN>(w, in, e, s); return;
+        case 2: go_gemv<T, 2, MODE, IN>(w, in, e, s); return;
+        default: go_gemv<T, 4, MODE, IN>(w, in, e, s); return;
+    }
 }
 
 template <typename T, DenseEpi MODE>
-void go(const DenseWeight& w, const void* a, uint32_t lda, uint32_t M, const DenseEpiArgs& e, hipStream_t s) {
+void go(const DenseWeight& w, const DenseIn& in, uint32_t M, const DenseEpiArgs& e, hipStream_t s) {
     if (M == 1) {
-        if constexpr (MODE != DenseEpi::Rope && MODE != DenseEpi::Split && MODE != DenseEpi::GateMul) {
-            switch (gemv_depth_split(w.N, w.K)) {
-                case 1: go_gemv<T, 1, MODE>(w, a, e, s); return;
-                case 2: go_gemv<T, 2, MODE>(w, a, e, s); return;
-                default: go_gemv<T, 4, MODE>(w, a, e, s); return;
-            }
-        }
+        if constexpr (MODE == DenseEpi::RawGate || MODE == DenseEpi::ActPair)
+            if (in.kind == DenseIn::Normed) { go_row<T, MODE, DenseIn::Normed>(w, in, e, s); return; }
+        if constexpr (MODE == DenseEpi::Residual)
+            if (in.kind == DenseIn::HeadGate) { go_row<T, MODE, DenseIn::HeadGate>(w, in, e, s); return; }
+        if constexpr (MODE != DenseEpi::Rope && MODE != DenseEpi::Split && MODE != DenseEpi::GateMul) { go_row<T, MODE, DenseIn::Rows>(w, in, e, s); return; }
     }
+    const void* a = in.rows;
+    const uint32_t lda = in.lda;
     // the large tile when its tiles give most compute units work, else the small one
     const uint64_t big = (uint64_t)((w.N + 127) / 128) * ((M + 127) / 128);
     if (big >= 192) go_gemm<T, 2, 2, MODE>(w, a, lda, M, e, s);
@@ -187,15 +280,15 @@ void go(const DenseWeight& w, const void* a, uint32_t lda, uint32_t M, const Den
 }
 
 template <typename T>
-void by_mode(const DenseWeight& w, const void* a, uint32_t lda, uint32_t M, DenseEpi mode, const DenseEpiArgs& e, hipStream_t s) {
+void by_mode(const DenseWeight& w, const DenseIn& in, uint32_t M, DenseEpi mode, const DenseEpiArgs& e, hipStream_t s) {
     switch (mode) {
-        case DenseEpi::F32: go<T, DenseEpi::F32>(w, a, lda, M, e, s); break;
-        case DenseEpi::RawGate: go<T, DenseEpi::RawGate>(w, a, lda, M, e, s); break;
-        case DenseEpi::Rope: go<T, DenseEpi::Rope>(w, a, lda, M, e, s); break;
-        case DenseEpi::Split: go<T, DenseEpi::Split>(w, a, lda, M, e, s); break;
-        case DenseEpi::GateMul: go<T, DenseEpi::GateMul>(w, a, lda, M, e, s); break;
-        case DenseEpi::SiluPair: go<T, DenseEpi::SiluPair>(w, a, lda, M, e, s); break;
-        case DenseEpi::Residual: go<T, DenseEpi::Residual>(w, a, lda, M, e, s); break;
+        case DenseEpi::F32: go<T, DenseEpi::F32>(w, in, M, e, s); break;
+        case DenseEpi::RawGate: go<T, DenseEpi::RawGate>(w, in, M, e, s); break;
+        case DenseEpi::Rope: go<T, DenseEpi::Rope>(w, in, M, e, s); break;
+        case DenseEpi::Split: go<T, DenseEpi::Split>(w, in, M, e, s); break;
+        case DenseEpi::GateMul: go<T, DenseEpi::GateMul>(w, in, M, e, s); break;
+        case DenseEpi::ActPair: go<T, DenseEpi::ActPair>(w, in, M, e, s); break;
+        case DenseEpi::Residual: go<T, DenseEpi::Residual>(w, in, M, e, s); break;
     }
 }
 
@@ -203,19 +296,37 @@ void by_mode(const DenseWeight& w, const void* a, uint32_t lda, uint32_t M, Dens
 
 uint32_t dense_k_max() { return DENSE_K_MAX; }
 
-void launch_dense(DType t, const DenseWeight& w, const void* a, uint32_t lda, uint32_t M, DenseEpi mode, const DenseEpiArgs& e, hipStream_t s) {
+void launch_dense(DType t, const DenseWeight& w, const DenseIn& in, uint32_t M, DenseEpi mode, const DenseEpiArgs& e, hipStream_t s) {
     if (M == 0 || w.N == 0) return;
-    if (t == DType::BF16) by_mode<__bf16>(w, a, lda, M, mode, e, s);
-    else by_mode<float>(w, a, lda, M, mode, e, s);
+    if (t == DType::BF16) by_mode<__bf16>(w, in, M, mode, e, s);
+    else by_mode<float>(w, in, M, mode, e, s);
 }
 
-void launch_dense_embedding(DType t, const void* table, uint32_t width, float scale, const uint32_t* tokens_dev, uint32_t M, float* x,
+namespace {
+
+template <typename T>
+void layer_norm(const float* x, uint32_t ldx, const LayerNorm& ln, uint32_t width, uint32_t M, void* out, uint32_t ld_out, hipStream_t s) {
+    auto go = [&](auto kernel) { fh::launch(kernel, dim3(M), 256, 0, s, x, ldx, ln, width, (T*)out, ld_out); };
+    if (width <= 1024) go(layer_norm_kernel<T, 1>);
+    else if (width <= 2048) go(layer_norm_kernel<T, 2>);
+    else if (width <= 4096) go(layer_norm_kernel<T, 4>);
+    else go(layer_norm_kernel<T, 16>);
+}
+
+}  // namespace
+
+void launch_layer_norm(DType t, const float* x, uint32_t ldx, const LayerNorm& ln, uint32_t width, uint32_t M, void* out, uint32_t ld_out, hipStream_t s) {
+    if (t == DType::BF16) layer_norm<__bf16>(x, ldx, ln, width, M, out, ld_out, s);
+    else layer_norm<float>(x, ldx, ln, width, M, out, ld_out, s);
+}
+
+void launch_dense_embedding(DType t, const void* table, uint32_t ld_table, uint32_t width, float scale, const uint32_t* tokens_dev, uint32_t M, float* x,
                             uint32_t ldx, const DynTanh& next, void* out, uint32_t ld_out, void* out2, uint32_t ld_out2, uint32_t* counts, hipStream_t s) {
     if (t == DType::BF16)
-        fh::launch(dense_embedding_kernel<__bf16>, dim3((ldx + 255) / 256, M), 256, 0, s, (const __bf16*)table, width, scale, tokens_dev, x, ldx, next, (__bf16*)out, ld_out,
+        fh::launch(dense_embedding_kernel<__bf16>, dim3((ldx + 255) / 256, M), 256, 0, s, (const __bf16*)table, ld_table, width, scale, tokens_dev, x, ldx, next, (__bf16*)out, ld_out,
                    (__bf16*)out2, ld_out2, counts);
     else
-        fh::launch(dense_embedding_kernel<float>, dim3((ldx + 255) / 256, M), 256, 0, s, (const float*)table, width, scale, tokens_dev, x, ldx, next, (float*)out, ld_out,
+        fh::launch(dense_embedding_kernel<float>, dim3((ldx + 255) / 256, M), 256, 0, s, (const float*)table, ld_table, width, scale, tokens_dev, x, ldx, next, (float*)out, ld_out,
                    (float*)out2, ld_out2, counts);
 }
 
