@@ -412,15 +412,49 @@ def vabirax_costs(cfg, prompt, context, es=2):
     return dec, pre
 
 
-def vabirax_bench(fh, args):
-    """--vabirax: prefill and decode throughput of the Vabirax design (random bfloat16 weights) at a size that resembles a real
-    model's layers, per stage against its roofline, and the Llama-family model of the same width, depth and feed-forward beside
-    it (Q8_0; its decode step both as a kernel sequence, the like of this design's, and as the resident kernel).  One JSON line."""
+def kakirax_costs(cfg, prompt, context, es=2):
+    """Per stage: bytes one decode step reads (and, for the states of linear attention, writes) at `context` cached positions, and
+    multiply-add operations of a prompt of `prompt` tokens (linear attention, as the recurrence: 4 per element of the state and token)."""
+    W, dec, pre = cfg["width"], {}, {}
+
+    def add(d, k, v):
+        d[k] = d.get(k, 0) + v
+
+    for layer in cfg["layers"]:
+        m, ff = layer["mixer"], (layer["mlp"] or {"ff": 0})["ff"]
+        H, d, dv = m["heads"], m["dim"], m["vdim"]
+        if layer["type"] == "attention":
+            G = m["kv_heads"]
+            proj = ((H + G) * d + (G + H) * dv) * W
+            add(dec, "attention", context * G * (d + dv) * es)
+            add(pre, "attention", 2 * (prompt * (prompt + 1) // 2) * H * (d + dv))
+        else:
+            rank = 16
+            proj = (2 * H * d + 2 * H * dv + rank) * W
+            add(dec, "attention", 2 * H * d * dv * 4 + rank * H * d * 4)
+            add(pre, "linear_attention", 4 * prompt * H * d * dv)
+        add(dec, "qkv_matmul", proj * es)
+        add(dec, "o_matmul", H * dv * W * es)
+        add(dec, "gate_up_matmul", 2 * ff * W * es)
+        add(dec, "down_matmul", ff * W * es)
+        add(pre, "qkv_matmul", 2 * prompt * proj)
+        add(pre, "o_matmul", 2 * prompt * H * dv * W)
+        add(pre, "gate_up_matmul", 4 * prompt * ff * W)
+        add(pre, "down_matmul", 2 * prompt * ff * W)
+    dec["lm_head_matmul"] = cfg["vocab"] * W * es
+    return dec, pre
+
+
+def folder_bench(fh, args, design, size, costs):
+    """--vabirax, --kakirax: prefill and decode throughput of a design that comes as a model folder (random bfloat16 weights) at a
+    size that resembles a real model's layers, per stage against its roofline, and the Llama-family model of the same width, depth
+    and feed-forward beside it (Q8_0; its decode step both as a kernel sequence, the like of this design's, and as the resident
+    kernel).  One JSON line."""
     import json as js
     import tempfile
     import numpy as np
     import torch
-    cfg = getattr(fh.synth, "vabirax_" + args.vabirax)()
+    cfg = getattr(fh.synth, design + "_" + size)()
     prompt = fh.synth.uniform_ids(args.seed + 1, args.prompt_tokens, cfg["vocab"])
     max_seq = (args.prompt_tokens + 2 * (args.warmup + args.steps) + 64 + 1023) // 1024 * 1024
 
@@ -446,6 +480,10 @@ def vabirax_bench(fh, args):
                 "decode_launches": model.decode_launches}, dec, pre, context
 
     def rooflines(dec, pre, dec_bytes, pre_ops, mfma_peak):
+        # linear attention shares the attention stage's clock; its products are 32-bit (157 TFLOP/s): counted at that rate
+        if "linear_attention" in pre_ops:
+            pre_ops = dict(pre_ops)
+            pre_ops["attention"] = pre_ops.get("attention", 0) + pre_ops.pop("linear_attention") * (2500 / 157)
         return ({s: {"us": round(dec[s][0], 1), "launches": dec[s][1], "GB/s": round(dec_bytes[s] / dec[s][0] / 1e3, 1),
                      "frac": round(dec_bytes[s] / dec[s][0] / 1e3 / 8000, 4)} for s in dec_bytes},
                 {s: {"ms": round(pre[s][0], 3), "TOP/s": round(pre_ops[s] / pre[s][0] / 1e9, 1),
@@ -453,7 +491,7 @@ def vabirax_bench(fh, args):
 
     with tempfile.TemporaryDirectory() as tmp:
         t0 = time.perf_counter()
-        fh.synth.write_model_folder(tmp, cfg, fh.synth.vabirax_stream(cfg, args.seed))
+        fh.synth.write_model_folder(tmp, cfg, fh.synth.folder_stream(cfg, args.seed))
         t_write = time.perf_counter() - t0
         print("written in %.1f s" % t_write, file=sys.stderr, flush=True)
         nbytes = os.path.getsize(os.path.join(tmp, "model.safetensors"))
@@ -463,15 +501,15 @@ def vabirax_bench(fh, args):
     print("loaded in %.1f s" % t_load, file=sys.stderr, flush=True)
     line, dec, pre, context = measure(model)
     model.close()
-    dec_bytes, pre_ops = vabirax_costs(cfg, len(prompt), context)
+    dec_bytes, pre_ops = costs(cfg, len(prompt), context)
     line["decode_stages"], line["prefill_stages"] = rooflines(dec, pre, dec_bytes, pre_ops, dict.fromkeys(pre_ops, 2500))
     line["decode_other_us"] = {s: round(v[0], 1) for s, v in dec.items() if s not in dec_bytes and v[1]}
     line["prefill_other_ms"] = {s: round(v[0], 3) for s, v in pre.items() if s not in pre_ops and v[1]}
 
     if args.no_closest:
-        print(js.dumps({"vabirax": line}))
+        print(js.dumps({design: line}))
         return
-    closest_name = {"135m": "smollm2_135m", "1b": "llama32_1b", "3b": "llama32_3b"}[args.vabirax]
+    closest_name = {"135m": "smollm2_135m", "1b": "llama32_1b", "3b": "llama32_3b"}[size]
     lcfg = getattr(fh.synth, closest_name)(fh.Q8_0, max_seq=max_seq)
     blob = fh.synth.make_weights_blob(lcfg, seed=args.seed, threads=16)
     print("Llama weights made", file=sys.stderr, flush=True)
@@ -492,12 +530,12 @@ def vabirax_bench(fh, args):
         model.close()
         gl["attention"] = L * context * 2 * KV * 2
         closest[name]["decode_stages"], closest[name]["prefill_stages"] = rooflines(dec, pre, gl, l_ops, peak)
-    print(js.dumps({"metric": "decode tok/s (Vabirax %s shape, bfloat16, 1 GPU)" % args.vabirax, "value": line["decode_tok_per_s"], "unit": "tok/s",
+    print(js.dumps({"metric": "decode tok/s (%s %s shape, bfloat16, 1 GPU)" % (design.capitalize(), size), "value": line["decode_tok_per_s"], "unit": "tok/s",
                     "n_gpus": 1, "steps": args.steps, "warmup": args.warmup, "ms_per_step": line["ms_per_step"], "higher_is_better": True,
                     "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
-                    "config": {"model": "Vabirax " + args.vabirax, "prompt_tokens": n, "weights_bytes": nbytes, "write_s": round(t_write, 1),
+                    "config": {"model": design.capitalize() + " " + size, "prompt_tokens": n, "weights_bytes": nbytes, "write_s": round(t_write, 1),
                                "load_s": round(t_load, 1)},
-                    "vabirax": line, "closest_model": {"model": closest_name + " shape, Q8_0", **closest}}))
+                    design: line, "closest_model": {"model": closest_name + " shape, Q8_0", **closest}}))
 
 
 def main():
@@ -522,9 +560,10 @@ def main():
                     help="length of the prompt (default: the 2502 tokens the metric is quoted on); the cache is sized to fit")
     ap.add_argument("--ops-table", action="store_true",
                     help="instead of the model benchmark, run the isolated kernels at the benchmark configurations' sizes")
-    ap.add_argument("--no-closest", action="store_true", help="with --vabirax: skip the Llama-family model")
+    ap.add_argument("--no-closest", action="store_true", help="with --vabirax or --kakirax: skip the Llama-family model")
     ap.add_argument("--vabirax", choices=("135m", "1b", "3b"),
                     help="instead of the default workload, the Vabirax design at this size beside the Llama-family model of the same size")
+    ap.add_argument("--kakirax", choices=("135m", "1b", "3b"), help="the same for the Kakirax design")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this build measures ONE GPU; --gpus must be 1 (no multi-GPU path exists to run)", file=sys.stderr)
@@ -538,7 +577,10 @@ def main():
         ops_table(fh)
         return
     if args.vabirax:
-        vabirax_bench(fh, args)
+        folder_bench(fh, args, "vabirax", args.vabirax, vabirax_costs)
+        return
+    if args.kakirax:
+        folder_bench(fh, args, "kakirax", args.kakirax, kakirax_costs)
         return
     wd = fh.Q8_0 if args.format == "q8_0" else fh.Q4_0
     PROMPT_TOKENS = args.prompt_tokens

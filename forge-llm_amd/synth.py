@@ -296,6 +296,61 @@ def vabirax_shapes(config) -> dict:
     return out
 
 
+def kakirax_attention(heads, kv_heads, dim, vdim, ff, scale=None, base=10000.0, rot_dims=None, scaling=None) -> dict:
+    """One attention entry of a Kakirax config's layer list; ff None: no feed-forward; scaling: (factor, low, high, original) or None."""
+    rot = {"base": base, "dims": rot_dims or dim}
+    if scaling:
+        rot["scaling"] = dict(zip(("factor", "low", "high", "original"), scaling))
+    return {"type": "attention", "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": dim ** -0.5 if scale is None else scale, "rot": rot},
+            "mlp": None if ff is None else {"kind": "dense", "ff": ff}}
+
+
+def kakirax_gla(heads, dim, vdim, ff, tau=16.0) -> dict:
+    """One gated-linear-attention entry of a Kakirax config's layer list."""
+    return {"type": "gla", "mixer": {"heads": heads, "dim": dim, "vdim": vdim, "tau": tau}, "mlp": None if ff is None else {"kind": "dense", "ff": ff}}
+
+
+def kakirax_config(width, vocab, layers, embedding_scale=1.0, eps=1e-5, cap=30.0) -> dict:
+    """layers: entries as above, or the index of the layer whose entry and weights a layer shares."""
+    layers = [dict(layers[x], weights_of=x) if isinstance(x, int) else x for x in layers]
+    return {"architecture": "Kakirax", "width": width, "vocab": vocab, "embedding": {"scale": embedding_scale}, "norm": {"eps": eps},
+            "logit_softcap": cap, "layers": layers}
+
+
+def kakirax_shapes(config, rank=16) -> dict:
+    """{tensor name: shape} of a Kakirax checkpoint; rank: of the decays' low-rank maps."""
+    w, out = config["width"], {}
+
+    def norm(name):
+        out[name], out[name + ".b"] = (w,), (w,)
+
+    out["embed"] = (config["vocab"], w)
+    for i, layer in enumerate(config["layers"]):
+        if layer.get("weights_of") is not None:
+            continue
+        m, n = layer["mixer"], "l%d." % i
+        H, d, dv = m["heads"], m["dim"], m["vdim"]
+        norm(n + "norm1")
+        if layer["type"] == "attention":
+            G = m["kv_heads"]
+            parts = (("q", (H * d, w)), ("k", (G * d, w)), ("v", (G * dv, w)), ("q.norm", (d,)), ("k.norm", (d,)), ("g", (H * dv, w)), ("o", (w, H * dv)))
+        else:
+            parts = (("q", (H * d, w)), ("k", (H * d, w)), ("v", (H * dv, w)), ("g", (H * dv, w)), ("o", (w, H * dv)), ("norm", (dv,)),
+                     ("a1", (rank, w)), ("a2", (H * d, rank)), ("a2.b", (H * d,)))
+        for name, shape in parts:
+            out[n + "mix." + name] = shape
+        if layer["mlp"] is not None:
+            norm(n + "norm2")
+            ff = layer["mlp"]["ff"]
+            out[n + "mlp.gate"], out[n + "mlp.up"], out[n + "mlp.down"] = (ff, w), (ff, w), (w, ff)
+    norm("final.norm")
+    return out
+
+
+def folder_shapes(config) -> dict:
+    return {"Vabirax": vabirax_shapes, "Kakirax": kakirax_shapes}[config["architecture"]](config)
+
+
 def to_bf16(x) -> np.ndarray:
     """float32 -> bfloat16 bits, to nearest even."""
     u = np.ascontiguousarray(x, np.float32).view(np.uint32).astype(np.uint64)
@@ -306,17 +361,19 @@ def from_bf16(bits) -> np.ndarray:
     return (np.asarray(bits, np.uint16).astype(np.uint32) << 16).view(np.float32)
 
 
-def vabirax_tensors(config, seed) -> dict:
-    """Random weights, bfloat16 bits by name: matrices with unit gain, norms that differ from element to element."""
+def folder_tensors(config, seed, shapes=None) -> dict:
+    """Random weights, bfloat16 bits by name: matrices with unit gain, norms that differ from element to element, decays from
+    almost none to strong."""
     rng = np.random.default_rng(seed)
     out = {}
-    for name, shape in vabirax_shapes(config).items():
+    shapes = shapes or folder_shapes(config)
+    for name, shape in shapes.items():
         if len(shape) == 2:
-            v = rng.standard_normal(shape) * (1.0 if name == "embed" else shape[1] ** -0.5)
+            v = rng.standard_normal(shape) * (1.0 if name == "embed" and "head" in shapes else shape[1] ** -0.5)
         elif name.endswith(".alpha"):
             v = rng.uniform(0.5, 1.2)
         elif name.endswith(".b"):
-            v = rng.standard_normal(shape) * 0.1
+            v = rng.standard_normal(shape) * (2.0 if name.endswith(".a2.b") else 0.1)
         else:
             v = rng.uniform(0.5, 1.5, shape)
         out[name] = to_bf16(np.asarray(v, np.float32)).reshape(shape)
@@ -348,7 +405,7 @@ def write_model_folder(path, config, tensors) -> None:
                 f.write(np.ascontiguousarray(t).tobytes())
 
 
-def vabirax_stream(config, seed) -> dict:
+def folder_stream(config, seed) -> dict:
     """Random weights for write_model_folder that are made while they are written: slices of one pool of normal numbers, scaled
     by the power of two nearest to unit gain.  For timing at real sizes."""
     rng = np.random.default_rng(seed)
@@ -366,9 +423,10 @@ def vabirax_stream(config, seed) -> dict:
         return write
 
     out = {}
-    for name, shape in vabirax_shapes(config).items():
+    shapes = folder_shapes(config)
+    for name, shape in shapes.items():
         if len(shape) == 2:
-            out[name] = (shape, matrix(shape, 0 if name == "embed" else int(round(np.log2(shape[1]) / 2))))
+            out[name] = (shape, matrix(shape, 0 if name == "embed" and "head" in shapes else int(round(np.log2(shape[1]) / 2))))
         else:
             out[name] = to_bf16(np.full(shape, 0.7 if name.endswith(".alpha") else 0.0 if name.endswith(".b") else 1.0, np.float32)).reshape(shape)
     return out
@@ -390,3 +448,24 @@ def vabirax_3b() -> dict:
     """Llama-3.2-3B's width, depth and feed-forward; 24 heads of 128 + 64 (values 128), latents of 1536 and 512."""
     layer = vabirax_layer(24, 128, 64, 128, 1536, 512, 8192, 4096, base=500000.0)
     return vabirax_config(3072, 128256, [layer] * 28, loop=(8, 20, 1), embedding_scale=1.0)
+
+
+def kakirax_sizes(width, vocab, depth, ff, attention, gla, embedding_scale, scaling) -> dict:
+    """Groups of three linear-attention layers and one attention layer, all with a feed-forward."""
+    layers = [kakirax_attention(*attention, ff, base=500000.0, scaling=scaling) if i % 4 == 3 else kakirax_gla(*gla, ff) for i in range(depth)]
+    return kakirax_config(width, vocab, layers, embedding_scale=embedding_scale)
+
+
+def kakirax_135m() -> dict:
+    """SmolLM2-135M's width, depth, feed-forward and attention; linear attention of 9 heads with keys of 32 and values of 64."""
+    return kakirax_sizes(576, 49152, 30, 1536, (9, 3, 64, 64), (9, 32, 64), 24.0, None)
+
+
+def kakirax_1b() -> dict:
+    """Llama-3.2-1B's width, depth, feed-forward and attention; linear attention of 16 heads with keys of 64 and values of 128."""
+    return kakirax_sizes(2048, 128256, 16, 8192, (32, 8, 64, 64), (16, 64, 128), 45.0, (32.0, 1.0, 4.0, 8192))
+
+
+def kakirax_3b() -> dict:
+    """Llama-3.2-3B's width, depth, feed-forward and attention; linear attention of 24 heads with keys of 64 and values of 128."""
+    return kakirax_sizes(3072, 128256, 28, 8192, (24, 8, 128, 128), (24, 64, 128), 55.0, (32.0, 1.0, 4.0, 8192))

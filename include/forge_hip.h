@@ -448,15 +448,18 @@ int32_t forge_hip_model_create_from_gguf(const char* path, uint32_t max_seq, uin
  * Designs that the reference does not have, described layer by layer in a config.json whose "architecture" picks an entry of the
  * library's registry (checkpoint.cpp): "Vabirax", a decoder of latent-attention layers (queries and keys / values through
  * low-rank latents, one rotated key part shared by all heads, a sliding window, a sigmoid gate on the heads' output) and gated
- * feed-forwards, Dynamic Tanh ahead of and behind every sublayer, part of the layers looped with a cache per pass.  The
+ * feed-forwards, Dynamic Tanh ahead of and behind every sublayer, part of the layers looped with a cache per pass; "Kakirax", a
+ * decoder that mixes layers of gated linear attention (a 32-bit state per head with a decay per key channel) and of grouped-query
+ * attention (normed queries and keys, rotation with stretched frequencies, an output gate), a layer norm ahead of every sublayer,
+ * layers that share weights, a capped output product with the embedding table.  The
  * handle is an ordinary model: forward, forward_greedy, prefill, profile, repeat penalty and reset work as documented above
- * (forge_hip_model_set_kv_pages and forge_hip_model_read_kv: this network has a flat cache of latents, they are refused).
+ * (forge_hip_model_set_kv_pages and forge_hip_model_read_kv: such networks have a flat cache of their own, they are refused).
  * dtype: FORGE_HIP_BF16 (weights, activations and cache in bfloat16, 32-bit sums; norms, rotation, scores, softmax and the
  * residual stream in 32-bit) or FORGE_HIP_F32 (everything in 32-bit).  max_seq = 0: 4096 positions.  flags: 0.
- * Limits: dim and rot_dim (each rounded up to 32) together at most 256, vdim at most 256, kv_rank at most 1024, width at most
- * 16384, heads * vdim and ff at most 32768; every other size is free. */
+ * Limits: dim and rot_dim (each rounded up to 32) together at most 256, vdim at most 256, kv_rank at most 1024, the decays' rank at
+ * most 128, width at most 16384, heads * vdim and ff at most 32768; every other size is free. */
 int32_t forge_hip_model_create_from_folder(const char* dir, uint32_t max_seq, uint32_t dtype, uint32_t flags, forge_hip_model** out);
-/* The sizes config.json gives, without a GPU (per-layer sizes: the first layer's; inter: the largest; max_seq and formats: 0). */
+/* The sizes config.json gives, without a GPU (per-layer sizes: the first attention layer's, or the first layer's; inter: the largest; max_seq and formats: 0). */
 int32_t forge_hip_folder_config(const char* dir, forge_hip_config* out);
 /* The configuration a handle was created with (any network). */
 int32_t forge_hip_model_config(const forge_hip_model* m, forge_hip_config* out);

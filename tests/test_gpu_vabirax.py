@@ -1,7 +1,4 @@
-"""The Vabirax network on the GPU, through the model handle, against the plain restatement in oracle/vabirax_oracle.py (64-bit).
-
-float32: every operation is single precision, so logits agree to a few 1e-6 of their size: a wrong key, norm or rotation has
-nowhere to hide.  bfloat16: the serving precision, held to the size of its rounding."""
+"""The Vabirax network on the GPU, through the model handle, against the plain restatement in oracle/vabirax_oracle.py (64-bit)."""
 import json
 import os
 import subprocess
@@ -10,29 +7,12 @@ import sys
 import numpy as np
 import pytest
 
+from folder_model import DTYPES, LIMIT, Case, check, decode_all, replay
 from vabirax_cases import cases
 
 pytestmark = pytest.mark.gpu
 
 NAMES = ["uneven", "many_heads", "wide_head", "large_rank", "ones", "no_window", "part_rotation"]
-LIMIT = {"float32": 3e-5, "bfloat16": 0.04}      # root mean square of a row's difference over that of all logits
-DTYPES = list(LIMIT)
-
-
-class Case:
-    """A configuration with random weights on disk, its oracle, and handles to it."""
-
-    def __init__(self, fh, vo, path, cfg, tensors=None, seed=5):
-        self.fh, self.cfg, self.path = fh, cfg, str(path)
-        self.tensors = tensors if tensors is not None else fh.synth.vabirax_tensors(cfg, seed)
-        fh.synth.write_model_folder(self.path, cfg, self.tensors)
-        self.oracle = vo.Oracle(cfg, {k: fh.synth.from_bf16(v) if v.dtype == np.uint16 else v for k, v in self.tensors.items()})
-
-    def model(self, max_seq=256, dtype="float32"):
-        return self.fh.HipModel.from_folder(self.path, max_seq, dtype)
-
-    def ids(self, n, seed=9):
-        return np.random.default_rng(seed).integers(0, self.cfg["vocab"], n)
 
 
 @pytest.fixture(scope="module")
@@ -51,17 +31,6 @@ def get(fh, vo, torch_gpu, tmp_path_factory):
             made[name] = Case(fh, vo, tmp_path_factory.mktemp(name), known[name])
         return made[name]
     return case
-
-
-def check(got, want, dtype, scale=None):
-    got, want = np.atleast_2d(np.asarray(got, np.float64)), np.atleast_2d(want)
-    assert np.all(np.isfinite(got))
-    err = np.sqrt(((got - want) ** 2).mean(axis=1)) / (scale or np.sqrt((want ** 2).mean()))
-    assert err.max() <= LIMIT[dtype], "row %d: %.3e" % (err.argmax(), err.max())
-
-
-def decode_all(model, ids):
-    return np.stack([model.forward(int(t)) for t in ids])
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
@@ -169,7 +138,7 @@ def needle_case(fh, vo, path, window, seed=3):
     token one key token takes nearly all the weight.  Returns the case, the query token, the key token and filler tokens with
     low scores."""
     cfg = fh.synth.vabirax_config(60, 80, [fh.synth.vabirax_layer(2, 24, 8, 20, 32, 40, None, window, scale=4.0)])
-    t = fh.synth.vabirax_tensors(cfg, seed)
+    t = fh.synth.folder_tensors(cfg, seed)
     uq = fh.synth.from_bf16(t["l0.mix.uq"]).reshape(2, 32, 32)
     uq[:, 24:] = 0.0
     uq[1] = uq[0]                                                         # both heads look for the same key
@@ -291,7 +260,7 @@ def test_mechanisms_alone(fh, vo, torch_gpu, tmp_path):
     lay = fh.synth.vabirax_layer(3, 12, 6, 10, 14, 18, 25, 11)
     cfg = fh.synth.vabirax_config(50, 60, [lay], embedding_scale=2.5, eps=0.02)
     looped = fh.synth.vabirax_config(50, 60, [lay], loop=(0, 1, 1), embedding_scale=2.5, eps=0.02)
-    base = fh.synth.vabirax_tensors(looped, 8)
+    base = fh.synth.folder_tensors(looped, 8)
     f = {k: fh.synth.from_bf16(v).astype(np.float64) for k, v in base.items()}
     norm = lambda x, n: vo.dyn_tanh(x, f[n + ".alpha"], f[n], f[n + ".b"])
     part = lambda prefix: {k[len(prefix):]: v for k, v in f.items() if k.startswith(prefix)}
@@ -442,7 +411,7 @@ def test_other_number_formats_and_refusals(get, fh, vo, tmp_path):
             fh.HipModel.from_folder(str(tmp_path / name), 64)
     big = json.loads(json.dumps(c.cfg))
     big["layers"][0]["mixer"]["kv_rank"] = 1100
-    fh.synth.write_model_folder(str(tmp_path / "big"), big, fh.synth.vabirax_tensors(big, 1))
+    fh.synth.write_model_folder(str(tmp_path / "big"), big, fh.synth.folder_tensors(big, 1))
     with pytest.raises(fh.ForgeHipError, match="kv_rank"):
         fh.HipModel.from_folder(str(tmp_path / "big"), 64)
 
@@ -461,27 +430,4 @@ def test_command_line(get):
 def test_trace_replay(get, tmp_path, dtype):
     """bin/trace_run on a small trace: two requests, one after the other, prompt portions and single tokens."""
     c = get("uneven")
-    root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
-    requests = {"a": c.ids(70, seed=71), "b": c.ids(33, seed=72)}
-    steps, expect = [], {}
-    for name, ids in requests.items():
-        want, at = c.oracle.forward(ids)[0], 0
-        for n in (40, 1, 2, 1, 1000):
-            n = min(n, ids.size - at)
-            if n <= 0:
-                break
-            rows = [] if n == 2 else sorted({0, n // 2, n - 1})[::-1]
-            expect[len(steps)] = want[[at + r for r in rows]]
-            steps.append({"step": len(steps), "entries": [{"id": name, "tokens": ids[at:at + n].tolist(), "want": rows}],
-                          "end": [name] if at + n == ids.size else []})
-            at += n
-    r = subprocess.run([sys.executable, os.path.join(root, "bin", "trace_run"), "--model", c.path, "--dtype", dtype, "--out", str(tmp_path), "--max-tokens", "128"],
-                       input="".join(json.dumps(s) + "\n" for s in steps), capture_output=True, text=True, timeout=100)
-    assert r.returncode == 0, r.stderr
-    assert [line for line in r.stdout.splitlines() if line.startswith("done")] == ["done %d" % i for i in range(len(steps))]
-    scale = np.sqrt((c.oracle.forward(requests["a"])[0] ** 2).mean())
-    for i, want in expect.items():
-        path = tmp_path / ("%d.f32" % i)
-        assert path.exists() == (want.size > 0)
-        if want.size:
-            check(np.fromfile(path, "<f4").reshape(want.shape), want, dtype, scale)
+    replay(c, {"a": c.ids(70, seed=71), "b": c.ids(33, seed=72)}, (40, 1, 2, 1, 1000), dtype, tmp_path)

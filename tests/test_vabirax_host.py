@@ -147,7 +147,7 @@ def test_norms(vo):
 
 def test_a_position_sees_nothing_later_and_nothing_before_its_windows(fh, vo):
     cfg = fh.synth.vabirax_config(24, 30, [fh.synth.vabirax_layer(2, 8, 4, 8, 12, 16, 20, 4)] * 2)
-    t = {k: fh.synth.from_bf16(v) for k, v in fh.synth.vabirax_tensors(cfg, 1).items()}
+    t = {k: fh.synth.from_bf16(v) for k, v in fh.synth.folder_tensors(cfg, 1).items()}
     o = vo.Oracle(cfg, t)
     ids = np.random.default_rng(2).integers(0, 30, 20)
     base = o.forward(ids)[0]
