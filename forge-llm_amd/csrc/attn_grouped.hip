@@ -14,54 +14,53 @@ constexpr float LOG2E = 1.4426950408889634f;
 constexpr float NO_KEYS = -3.0e38f;          // maximum of a part without keys: weight 0
 constexpr uint32_t GA_NW = 4, GA_KT = 16 * GA_NW, GA_SPLITS_MAX = 64;
 
-// One head of `dim` raw elements by one wave: norm, rotation of the pairs (2 i, 2 i + 1), i < pairs, store as T.
-template <typename T>
-__device__ __forceinline__ void norm_rotate_head(const float* __restrict__ raw, const float* __restrict__ w, uint32_t dim, uint32_t dim_n, float eps,
-                                                 const float* __restrict__ ct, const float* __restrict__ st, uint32_t pairs, T* out, uint32_t lane) {
-    constexpr uint32_t NP = DENSE_HEAD_MAX / 128;
-    float2 v[NP];
-    float ss = 0.f;
-#pragma unroll
-    for (uint32_t i = 0; i < NP; i++) {
-        const uint32_t p = lane + 64 * i;
-        v[i] = 2 * p < dim ? *reinterpret_cast<const float2*>(raw + 2 * p) : make_float2(0.f, 0.f);      // zero past dim_n
-        ss = fmaf(v[i].x, v[i].x, ss);
-        ss = fmaf(v[i].y, v[i].y, ss);
-    }
-    const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)dim_n + eps);
-#pragma unroll
-    for (uint32_t i = 0; i < NP; i++) {
-        const uint32_t p = lane + 64 * i;
-        if (2 * p >= dim) continue;
-        const float2 nw = *reinterpret_cast<const float2*>(w + 2 * p);
-        float a = v[i].x * inv * nw.x, b = v[i].y * inv * nw.y;
-        if (p < pairs) {
-            const float c = ct[p], s = st[p];
-            const float a2 = a * c - b * s;
-            b = b * c + a * s;
-            a = a2;
-        }
-        struct __attribute__((aligned(2 * sizeof(T)))) Pair { T a, b; } r = {(T)a, (T)b};
-        *reinterpret_cast<Pair*>(out + 2 * p) = r;
-    }
+// Sum over groups of LANES lanes.
+template <int LANES> __device__ __forceinline__ float group_sum(float v) {
+    static_assert(LANES == 16 || LANES == 32 || LANES == 64, "power of two up to the wave");
+    if (LANES >= 64) v = lane_xor_add<32>(v);
+    if (LANES >= 32) v = lane_xor_add<16>(v);
+    return lane_xor_add<1>(lane_xor_add<2>(lane_xor_add<4>(lane_xor_add<8>(v))));
 }
 
-// One workgroup per row: a wave takes every fourth head.
-template <typename T>
+// One head of `dim` raw elements by a group of LANES >= dim / 4 lanes, of which this one is number `sub`: norm, rotation of the pairs
+// (2 i, 2 i + 1), i < pairs, store as T.
+template <typename T, int LANES>
+__device__ __forceinline__ void norm_rotate_head(const float* __restrict__ raw, const float* __restrict__ w, uint32_t dim, uint32_t dim_n, float eps,
+                                                 const float* __restrict__ ct, const float* __restrict__ st, uint32_t pairs, T* out, uint32_t sub) {
+    const bool in = 4 * sub < dim;
+    v4f v = (v4f){0.f, 0.f, 0.f, 0.f}, nw = v;
+    float c[2] = {1.f, 1.f}, s[2] = {0.f, 0.f};
+    if (in) {
+        v = *reinterpret_cast<const v4f*>(raw + 4 * sub);                // zero past dim_n
+        nw = *reinterpret_cast<const v4f*>(w + 4 * sub);
+#pragma unroll
+        for (uint32_t i = 0; i < 2; i++)
+            if (2 * sub + i < pairs) { c[i] = ct[2 * sub + i]; s[i] = st[2 * sub + i]; }
+    }
+    const float inv = 1.0f / sqrtf(group_sum<LANES>((v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3])) / (float)dim_n + eps);
+    if (!in) return;
+    v *= inv;
+    v *= nw;
+    store4<T>(out + 4 * sub, v[0] * c[0] - v[1] * s[0], v[1] * c[0] + v[0] * s[0], v[2] * c[1] - v[3] * s[1], v[3] * c[1] + v[2] * s[1]);
+}
+
+// One workgroup per row: 256 / LANES heads at a time.
+template <typename T, int LANES>
 __global__ __launch_bounds__(256) void grouped_norm_store_kernel(GroupedShape sh, const float* __restrict__ raw, const float* __restrict__ q_norm,
                                                                  const float* __restrict__ k_norm, const float* __restrict__ cos_t,
                                                                  const float* __restrict__ sin_t, uint32_t base_pos, T* __restrict__ q,
                                                                  T* __restrict__ kc, T* __restrict__ vc) {
-    const uint32_t m = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, pos = base_pos + m;
+    const uint32_t m = blockIdx.x, tid = threadIdx.x, sub = tid % LANES, pos = base_pos + m;
     const float* row = raw + (size_t)m * sh.raw_row();
     const float* ct = cos_t + (size_t)pos * sh.rot_pairs;
     const float* st = sin_t + (size_t)pos * sh.rot_pairs;
-    for (uint32_t h = wave; h < sh.heads; h += 4)
-        norm_rotate_head<T>(row + h * sh.dim, q_norm, sh.dim, sh.dim_n, sh.eps, ct, st, sh.rot_pairs, q + ((size_t)m * sh.heads + h) * sh.dim, lane);
-    const float* kr = row + sh.heads * sh.dim;
-    for (uint32_t g = wave; g < sh.kv_heads; g += 4)
-        norm_rotate_head<T>(kr + g * sh.dim, k_norm, sh.dim, sh.dim_n, sh.eps, ct, st, sh.rot_pairs, kc + (size_t)pos * sh.k_row() + g * sh.dim, lane);
-    const float* vr = kr + sh.k_row();
+    // the keys' heads follow the queries'
+    for (uint32_t h = tid / LANES; h < sh.heads + sh.kv_heads; h += 256 / LANES) {
+        const bool query = h < sh.heads;
+        T* out = query ? q + ((size_t)m * sh.heads + h) * sh.dim : kc + (size_t)pos * sh.k_row() + (h - sh.heads) * sh.dim;
+        norm_rotate_head<T, LANES>(row + h * sh.dim, query ? q_norm : k_norm, sh.dim, sh.dim_n, sh.eps, ct, st, sh.rot_pairs, out, sub);
+    }
+    const float* vr = row + (sh.heads + sh.kv_heads) * sh.dim;
     for (uint32_t i = tid * 4; i < sh.v_row(); i += 1024) {
         const float4 v = *reinterpret_cast<const float4*>(vr + i);
         store4<T>(vc + (size_t)pos * sh.v_row() + i, v.x, v.y, v.z, v.w);
@@ -79,6 +78,7 @@ __global__ __launch_bounds__(GA_NW * 64) void grouped_decode_kernel(GroupedShape
                                                                     uint32_t base_pos, const uint32_t* __restrict__ pos_dev) {
     typedef typename Vec<T>::x8 x8;
     constexpr uint32_t NW = GA_NW, KT = GA_KT, PAD = 16 / sizeof(T), VS = KT + PAD, MAXT = (2 * DV + NW - 1) / NW;
+    constexpr uint32_t LANES = 8 * DK;                      // that norm one head
     extern __shared__ __attribute__((aligned(16))) uint8_t ga_lds[];
     const uint32_t QS = sh.dim + PAD;
     T* Vt = reinterpret_cast<T*>(ga_lds);                   // [vdim][VS]
@@ -118,15 +118,17 @@ __global__ __launch_bounds__(GA_NW * 64) void grouped_decode_kernel(GroupedShape
     const float* st = sin_t + (size_t)pos * sh.rot_pairs;
     if (fresh) {
         const float* kr = raw + sh.heads * sh.dim;
-        if (wave == NW - 1) norm_rotate_head<T>(kr + kvh * sh.dim, k_norm, sh.dim, sh.dim_n, sh.eps, ct, st, sh.rot_pairs, kc + (size_t)pos * sh.k_row() + kvh * sh.dim, lane);
+        if (wave == NW - 1 && lane < LANES)
+            norm_rotate_head<T, LANES>(kr + kvh * sh.dim, k_norm, sh.dim, sh.dim_n, sh.eps, ct, st, sh.rot_pairs, kc + (size_t)pos * sh.k_row() + kvh * sh.dim, lane);
         const float* vr = kr + sh.k_row() + kvh * sh.vdim;
         if (wave == NW - 2)
             for (uint32_t i = lane; i < sh.vdim; i += 64) vc[(size_t)pos * sh.v_row() + kvh * sh.vdim + i] = (T)vr[i];
     }
-    for (uint32_t h = wave; h < 16; h += NW) {
-        if (h < nh) norm_rotate_head<T>(raw + (h0 + h) * sh.dim, q_norm, sh.dim, sh.dim_n, sh.eps, ct, st, sh.rot_pairs, Q + h * QS, lane);
-        else
-            for (uint32_t i = lane; i < sh.dim; i += 64) Q[h * QS + i] = (T)0.f;
+#pragma unroll
+    for (uint32_t i = 0; i < 16 * LANES / (NW * 64); i++) {
+        const uint32_t h = tid / LANES + i * (NW * 64 / LANES), sub = tid % LANES;
+        if (h < nh) norm_rotate_head<T, LANES>(raw + (h0 + h) * sh.dim, q_norm, sh.dim, sh.dim_n, sh.eps, ct, st, sh.rot_pairs, Q + h * QS, sub);
+        else if (4 * sub < sh.dim) store4<T>(Q + h * QS + 4 * sub, 0.f, 0.f, 0.f, 0.f);
     }
     __syncthreads();
     if (!early) fetch(t0);
@@ -256,8 +258,12 @@ void decode(const GroupedShape& sh, const GroupedIo& io, float* parts, const voi
 
 template <typename T>
 void norm_store(const GroupedShape& sh, const GroupedIo& io, uint32_t M, void* q, hipStream_t s) {
-    fh::launch(grouped_norm_store_kernel<T>, dim3(M), 256, 0, s, sh, io.raw, io.q_norm, io.k_norm, io.cos_t, io.sin_t, io.base_pos, (T*)q, (T*)io.k_cache,
-               (T*)io.v_cache);
+    auto go = [&](auto kernel) {
+        fh::launch(kernel, dim3(M), 256, 0, s, sh, io.raw, io.q_norm, io.k_norm, io.cos_t, io.sin_t, io.base_pos, (T*)q, (T*)io.k_cache, (T*)io.v_cache);
+    };
+    if (sh.dim <= 64) go(grouped_norm_store_kernel<T, 16>);
+    else if (sh.dim <= 128) go(grouped_norm_store_kernel<T, 32>);
+    else go(grouped_norm_store_kernel<T, 64>);
 }
 
 }  // namespace

@@ -358,7 +358,7 @@ struct LinearMixer : Mixer {
         sh.heads = a.heads;
         sh.dim = pad_to(a.dim, 32);
         sh.vdim = pad_to(a.vdim, 32);
-        sh.rank = pad_to(rank, 32);
+        sh.rank = pad_to(rank, 16);
         sh.vdim_n = a.vdim;
         sh.q_scale = (float)(1.0 / sqrt((double)a.dim));
         sh.inv_tau = (float)(1.0 / a.tau);

@@ -384,7 +384,7 @@ void launch_grouped_decode(DType t, const GroupedShape& sh, const GroupedIo& io,
 // per key channel a = sigmoid(W2 low + b)^(1 / tau).  All of it in 32-bit for both element types.  Padded sizes (multiples of 32).
 struct LinearShape {
     uint32_t heads = 0, dim = 0, vdim = 0;
-    uint32_t rank = 0;                       // of the decay's low-rank map (a multiple of 4)
+    uint32_t rank = 0;                       // of the decay's low-rank map (a multiple of 16)
     uint32_t vdim_n = 0;                     // elements a head's output norm counts
     float q_scale = 0.f, inv_tau = 0.f, eps = 0.f;
     __host__ __device__ uint32_t qk() const { return heads * dim; }

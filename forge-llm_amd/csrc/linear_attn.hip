@@ -21,7 +21,7 @@ namespace fh {
 constexpr uint32_t LA_CHUNK = 64, LA_PIECE = 16, LA_PIECES = LA_CHUNK / LA_PIECE;
 constexpr uint32_t LA_LS = LA_CHUNK + 4;     // LDS row stride in floats
 constexpr uint32_t LA_MAX = 256;             // dim and vdim
-constexpr uint32_t LA_RANK_MAX = 128;
+constexpr uint32_t LA_RANK_MAX = 128, LA_RANK_STEP = 16;
 
 __device__ __forceinline__ float decay_of(float z, float inv_tau) {
     // log sigmoid(z) = min(z, 0) - log(1 + e^-|z|)
@@ -77,11 +77,18 @@ __global__ __launch_bounds__(256) void linear_step_kernel(LinearShape sh, const 
 }
 
 // ---- prompt -------------------------------------------------------------------------------------------------------------------
-// Eight values of one column, rows t .. t + 7 of a matrix in memory (zero from row `rows` on).
-__device__ __forceinline__ v8f column8(const float* __restrict__ p, size_t ld, uint32_t t, uint32_t rows) {
+// `rows` rows of `width` floats, ld apart, as a buffer: what lies past the last row reads as zero.  Offsets are in bytes.
+__device__ __forceinline__ __amdgpu_buffer_rsrc_t rows_buffer(const float* p, uint32_t rows, uint32_t ld, uint32_t width) {
+    return __builtin_amdgcn_make_buffer_rsrc((void*)p, 0, ((rows - 1) * ld + width) * 4, 0x00020000);
+}
+__device__ __forceinline__ float buffer_float(__amdgpu_buffer_rsrc_t b, uint32_t offset) {
+    return __builtin_bit_cast(float, __builtin_amdgcn_raw_buffer_load_b32(b, offset, 0, 0));
+}
+// Eight values of one column, `step` bytes apart.
+__device__ __forceinline__ v8f column8(__amdgpu_buffer_rsrc_t b, uint32_t offset, uint32_t step) {
     v8f f;
 #pragma unroll
-    for (uint32_t e = 0; e < 8; e++) f[e] = t + e < rows ? p[(t + e) * ld] : 0.f;
+    for (uint32_t e = 0; e < 8; e++) f[e] = buffer_float(b, offset + e * step);
     return f;
 }
 
@@ -92,11 +99,34 @@ __global__ __launch_bounds__(256) void linear_chunk_kernel(LinearShape sh, const
     float* kt = lc_lds;                                       // [dim][LA_LS]: keys, decayed to their piece's end
     float* low = kt + sh.dim * LA_LS;                         // [64][rank + 4]
     float* dp = low + LA_CHUNK * (sh.rank + 4);               // [4][dim]: decay of a piece, then of all pieces behind it
-    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, lq = lane & 31, lh = lane >> 5;
-    const uint32_t chunk = blockIdx.x, head = blockIdx.y, m0 = chunk * LA_CHUNK, rows = min(M - m0, LA_CHUNK), LR = sh.rank + 4;
-    const size_t ld = sh.raw_row();
+    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = (uint32_t)__builtin_amdgcn_readfirstlane((int)(tid >> 6)), lq = lane & 31, lh = lane >> 5;
+    const uint32_t chunk = blockIdx.x, head = blockIdx.y, m0 = chunk * LA_CHUNK, rows = min(M - m0, LA_CHUNK), LR = sh.rank + 4, ld = sh.raw_row();
     const float* r0 = raw + (size_t)m0 * ld;
     const float* lowp = r0 + 2 * sh.qk() + sh.heads * sh.vdim;
+    const uint32_t nv = sh.vdim / 32, n = nv * (sh.dim / 32);
+    // the values of a tile; the wave's first are requested ahead of everything
+    v8f vf[LA_PIECES];
+    const __amdgpu_buffer_rsrc_t vbuf = rows_buffer(r0 + 2 * sh.qk() + head * sh.vdim, rows, ld, sh.vdim);
+    auto fetch_values = [&](uint32_t i) {
+#pragma unroll
+        for (uint32_t s = 0; s < LA_PIECES; s++) vf[s] = column8(vbuf, ((16 * s + 8 * lh) * ld + i % nv * 32 + lq) * 4, ld * 4);
+    };
+    fetch_values(wave);
+    // the keys of a channel over one piece, and the first of its row of the map
+    const __amdgpu_buffer_rsrc_t kbuf = rows_buffer(r0 + sh.qk() + head * sh.dim, rows, ld, sh.dim);
+    float k[LA_PIECE], w[LA_RANK_STEP], b;
+    auto fetch_map = [&](uint32_t ch, uint32_t r) {
+#pragma unroll
+        for (uint32_t j = 0; j < LA_RANK_STEP; j++) w[j] = w2[(size_t)(r + j) * sh.qk() + ch];
+    };
+    auto fetch_channel = [&](uint32_t i) {
+        const uint32_t c = i % sh.dim, t0 = i / sh.dim * LA_PIECE;
+#pragma unroll
+        for (uint32_t t = 0; t < LA_PIECE; t++) k[t] = buffer_float(kbuf, ((t0 + t) * ld + c) * 4);
+        fetch_map(head * sh.dim + c, 0);
+        b = b2[head * sh.dim + c];
+    };
+    if (tid < LA_PIECES * sh.dim) fetch_channel(tid);
     for (uint32_t i = tid; i < LA_CHUNK * (sh.rank / 4); i += 256) {
         const uint32_t t = i / (sh.rank / 4), c = i % (sh.rank / 4) * 4;
         *reinterpret_cast<v4f*>(low + t * LR + c) = t < rows ? *reinterpret_cast<const v4f*>(lowp + t * ld + c) : (v4f){0.f, 0.f, 0.f, 0.f};
@@ -104,23 +134,20 @@ __global__ __launch_bounds__(256) void linear_chunk_kernel(LinearShape sh, const
     __syncthreads();
     for (uint32_t i = tid; i < LA_PIECES * sh.dim; i += 256) {
         const uint32_t c = i % sh.dim, piece = i / sh.dim, ch = head * sh.dim + c, t0 = piece * LA_PIECE;
-        float k[LA_PIECE], z[LA_PIECE];
-        const float b = b2[ch];
+        float z[LA_PIECE];
+        if (i != tid) fetch_channel(i);
 #pragma unroll
-        for (uint32_t t = 0; t < LA_PIECE; t++) {
-            k[t] = t0 + t < rows ? r0[(t0 + t) * ld + sh.qk() + ch] : 0.f;
-            z[t] = b;
-        }
-        for (uint32_t r = 0; r < sh.rank; r += 4) {
-            float w[4];
+        for (uint32_t t = 0; t < LA_PIECE; t++) z[t] = b;
+        for (uint32_t r = 0; r < sh.rank; r += LA_RANK_STEP) {
+            if (r) fetch_map(ch, r);
 #pragma unroll
-            for (int j = 0; j < 4; j++) w[j] = w2[(size_t)(r + j) * sh.qk() + ch];
+            for (uint32_t t = 0; t < LA_PIECE; t++)
 #pragma unroll
-            for (uint32_t t = 0; t < LA_PIECE; t++) {
-                const v4f l = *reinterpret_cast<const v4f*>(low + (t0 + t) * LR + r);
+                for (uint32_t g = 0; g < LA_RANK_STEP; g += 4) {
+                    const v4f l = *reinterpret_cast<const v4f*>(low + (t0 + t) * LR + r + g);
 #pragma unroll
-                for (int j = 0; j < 4; j++) z[t] = fmaf(w[j], l[j], z[t]);
-            }
+                    for (uint32_t j = 0; j < 4; j++) z[t] = fmaf(w[g + j], l[j], z[t]);
+                }
         }
 #pragma unroll
         for (uint32_t t = 0; t < LA_PIECE; t++) {
@@ -146,67 +173,66 @@ __global__ __launch_bounds__(256) void linear_chunk_kernel(LinearShape sh, const
         total[(size_t)chunk * sh.qk() + head * sh.dim + c] = p;
     }
     __syncthreads();
-    const uint32_t nv = sh.vdim / 32, n = nv * (sh.dim / 32);
     for (uint32_t i = wave; i < n; i += 4) {
         const uint32_t ct = i / nv * 32, vt = i % nv * 32;
-        const float* v = r0 + 2 * sh.qk() + head * sh.vdim + vt + lq;
         v16f acc;
 #pragma unroll
         for (int r = 0; r < 16; r++) acc[r] = 0.f;
 #pragma unroll
         for (uint32_t s = 0; s < LA_PIECES; s++) {
             const v8f a = load8(kt + (ct + lq) * LA_LS + 16 * s + 8 * lh) * dp[s * sh.dim + ct + lq];
-            acc = mma32(a, column8(v, ld, 16 * s + 8 * lh, rows), acc);
+            acc = mma32(a, vf[s], acc);
         }
+        if (i + 4 < n) fetch_values(i + 4);
         float* y = add + (((size_t)chunk * sh.heads + head) * sh.dim + ct) * sh.vdim + vt + lq;
 #pragma unroll
         for (int r = 0; r < 16; r++) y[(size_t)(8 * (r >> 2) + 4 * lh + (r & 3)) * sh.vdim] = acc[r];
     }
 }
 
-// add[chunk] <- the state ahead of the chunk; state <- the one behind the last.  A thread owns two neighbouring elements.
+// add[chunk] <- the state ahead of the chunk; state <- the one behind the last.  A thread owns one element.
 __global__ __launch_bounds__(256) void linear_scan_kernel(LinearShape sh, uint32_t chunks, const float* __restrict__ total, float* add, float* state, uint32_t base_pos) {
-    const size_t n = sh.state(), i = ((size_t)blockIdx.x * 256 + threadIdx.x) * 2;
+    const size_t n = sh.state(), i = (size_t)blockIdx.x * 256 + threadIdx.x;
     if (i >= n) return;
     const float* d = total + i / sh.vdim;
-    float2 s = base_pos ? *reinterpret_cast<const float2*>(state + i) : make_float2(0.f, 0.f);
-    constexpr uint32_t B = 8;
+    float s = base_pos ? state[i] : 0.f;
+    constexpr uint32_t B = 16;
     for (uint32_t c0 = 0; c0 < chunks; c0 += B) {
-        float2 x[B];
-        float f[B];
+        float x[B], f[B];
 #pragma unroll
         for (uint32_t b = 0; b < B; b++) {
             const uint32_t c = min(c0 + b, chunks - 1);
-            x[b] = *reinterpret_cast<const float2*>(add + c * n + i);
+            x[b] = add[c * n + i];
             f[b] = d[(size_t)c * sh.qk()];
         }
 #pragma unroll
         for (uint32_t b = 0; b < B; b++) {
             if (c0 + b >= chunks) break;
-            *reinterpret_cast<float2*>(add + (c0 + b) * n + i) = s;
-            s.x = fmaf(f[b], s.x, x[b].x);
-            s.y = fmaf(f[b], s.y, x[b].y);
+            add[(c0 + b) * n + i] = s;
+            s = fmaf(f[b], s, x[b]);
         }
     }
-    *reinterpret_cast<float2*>(state + i) = s;
+    state[i] = s;
 }
 
 // Workgroup = (chunk, head), key channels 64 at a time.  A wave owns one piece of 16 tokens (loading, its own pairs, the running
 // products), then its share of the pieces' pairs and of the output tiles.  Outputs are computed transposed: a lane owns one token.
 // TILES: output tiles of a wave, at least.
 template <typename T, int TILES>
-__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void linear_output_kernel(LinearShape sh, const float* __restrict__ raw, const float* __restrict__ decay, const float* __restrict__ before,
+__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(TILES <= 2 ? 3 : 2))) void linear_output_kernel(LinearShape sh, const float* __restrict__ raw, const float* __restrict__ decay, const float* __restrict__ before,
                                                             uint32_t M, const float* __restrict__ norm, const T* __restrict__ gate, T* __restrict__ out, uint32_t ld_out) {
     __shared__ __attribute__((aligned(16))) float qs[LA_CHUNK * LA_LS], ks[LA_CHUNK * LA_LS], ps[LA_CHUNK * LA_LS];    // ps: decays, then the pairs' weights
     __shared__ __attribute__((aligned(16))) float ahead[LA_PIECES][64], between[3][64];      // decay of the pieces ahead in the chunk; of piece 1, of 2, of both
     typedef typename Vec<T>::x4 x4;
     constexpr uint32_t LS = LA_LS;
-    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, lq = lane & 31, lh = lane >> 5, l16 = lane & 15, lg = lane >> 4;
-    const uint32_t chunk = blockIdx.x, head = blockIdx.y, m0 = chunk * LA_CHUNK, rows = min(M - m0, LA_CHUNK);
-    const size_t ld = sh.raw_row();
+    constexpr int EARLY = 1;                                 // output tiles whose operands are requested early
+    const uint32_t tid = threadIdx.x, wave = (uint32_t)__builtin_amdgcn_readfirstlane((int)(tid >> 6));
+    uint32_t lane = tid & 63;
+    const uint32_t chunk = blockIdx.x, head = blockIdx.y, m0 = chunk * LA_CHUNK, rows = min(M - m0, LA_CHUNK), ld = sh.raw_row();
     const float* r0 = raw + (size_t)m0 * ld;
     const uint32_t nv = sh.vdim / 32, ntile = 2 * nv;        // tile i: value columns i % nv, tokens 32 (i / nv) ..
     const float* S = before + ((size_t)chunk * sh.heads + head) * sh.dim * sh.vdim;
+    const __amdgpu_buffer_rsrc_t vbuf = rows_buffer(r0 + 2 * sh.qk() + head * sh.vdim, rows, ld, sh.vdim);
 
     v16f acc[TILES];
 #pragma unroll
@@ -220,18 +246,37 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void l
     constexpr uint32_t LATER = 0x332321, EARLIER = 0x010210, BETWEEN = 0x210333;
 
     for (uint32_t s0 = 0; s0 < sh.dim; s0 += 64) {
-        const uint32_t sw = min(64u, sh.dim - s0);
+        asm volatile("" : "+v"(lane));                       // else the offsets of all loads stay in registers from pass to pass
+        const uint32_t sw = min(64u, sh.dim - s0), lq = lane & 31, lh = lane >> 5, l16 = lane & 15, lg = lane >> 4;
         {
-            const float* qp = r0 + wave * LA_PIECE * ld + head * sh.dim + s0 + lane;
-            const float* ap = decay + (size_t)(m0 + wave * LA_PIECE) * sh.qk() + head * sh.dim + s0 + lane;
-#pragma unroll 4
-            for (uint32_t m = wave * LA_PIECE; m < (wave + 1) * LA_PIECE; m++, qp += ld, ap += sh.qk()) {
-                const bool in = m < rows && lane < sw;
-                qs[m * LS + lane] = in ? qp[0] * sh.q_scale : 0.f;
-                ks[m * LS + lane] = in ? qp[sh.qk()] : 0.f;
-                ps[m * LS + lane] = in ? ap[0] : 1.f;
+            // past the last token, and past the head's channels, all three are zero
+            const __amdgpu_buffer_rsrc_t qb = rows_buffer(r0 + head * sh.dim + s0, rows, ld, sw), kb = rows_buffer(r0 + sh.qk() + head * sh.dim + s0, rows, ld, sw),
+                                         ab = rows_buffer(decay + (size_t)m0 * sh.qk() + head * sh.dim + s0, rows, sh.qk(), sw);
+            const uint32_t out_of_range = lane < sw ? 0 : 0x40000000;
+            const uint32_t q0 = (wave * LA_PIECE * ld + lane) * 4 + out_of_range, a0 = (wave * LA_PIECE * sh.qk() + lane) * 4 + out_of_range;
+            float q[LA_PIECE], k[LA_PIECE], a[LA_PIECE];
+#pragma unroll
+            for (uint32_t i = 0; i < LA_PIECE; i++) {
+                q[i] = buffer_float(qb, q0 + i * ld * 4) * sh.q_scale;
+                k[i] = buffer_float(kb, q0 + i * ld * 4);
+                a[i] = buffer_float(ab, a0 + i * sh.qk() * 4);
+            }
+#pragma unroll
+            for (uint32_t i = 0; i < LA_PIECE; i++) {
+                const uint32_t at = (wave * LA_PIECE + i) * LS + lane;
+                qs[at] = q[i];
+                ks[at] = k[i];
+                ps[at] = a[i];
             }
         }
+        // the state ahead of the chunk, for the output tiles: requested ahead of the pairs
+        const __amdgpu_buffer_rsrc_t sbuf = rows_buffer(S + (size_t)s0 * sh.vdim, sw, sh.vdim, sh.vdim);
+        auto state8 = [&](uint32_t n, uint32_t s) { return column8(sbuf, ((s + 8 * lh) * sh.vdim + n % nv * 32 + lq) * 4, sh.vdim * 4); };
+        v8f sf[EARLY][4];
+#pragma unroll
+        for (int i = 0; i < EARLY; i++)
+#pragma unroll
+            for (uint32_t s = 0; s < 4; s++) sf[i][s] = state8(wave + 4 * i, 16 * s);
         __syncthreads();
         {
             const uint32_t j = lane >> 2, at = wave * LA_PIECE * LS + (lane & 3) * 16;
@@ -305,16 +350,24 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void l
             const uint32_t n = wave + 4 * i;
             if (n >= ntile) continue;
             const uint32_t t = n / nv * 32 + lq;
-            const float* sp = S + (size_t)s0 * sh.vdim + n % nv * 32 + lq;
-#pragma unroll 2
-            for (uint32_t s = 0; s < sw; s += 16) {
+#pragma unroll
+            for (uint32_t s = 0; s < 64; s += 16) {
+                if (s >= sw) break;
                 const v8f q = load8(qs + t * LS + s + 8 * lh) * load8(&ahead[t / LA_PIECE][s + 8 * lh]);
-                acc[i] = mma32(column8(sp, sh.vdim, s + 8 * lh, sw), q, acc[i]);
+                acc[i] = mma32(i < EARLY ? sf[i < EARLY ? i : 0][s / 16] : state8(n, s), q, acc[i]);
+                __builtin_amdgcn_sched_barrier(0);           // operands of a later step would take registers now
             }
         }
         __syncthreads();
     }
 
+    const uint32_t lq = lane & 31, lh = lane >> 5, l16 = lane & 15, lg = lane >> 4;
+    auto values8 = [&](uint32_t n, uint32_t s) { return column8(vbuf, ((s + 8 * lh) * ld + n % nv * 32 + lq) * 4, ld * 4); };
+    v8f vf[EARLY][4];                                        // the chunk's values, for the first tiles
+#pragma unroll
+    for (int i = 0; i < EARLY; i++)
+#pragma unroll
+        for (uint32_t s = 0; s < 4; s++) vf[i][s] = values8(wave + 4 * i, 16 * s);
     // the weights of all pairs (t, j), j <= t
 #pragma unroll
     for (uint32_t i = 0; i < LA_PIECE / 4; i++) ps[(wave * LA_PIECE + (lane & 3) + 4 * i) * LS + wave * LA_PIECE + (lane >> 2)] = own[i];
@@ -334,9 +387,12 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void l
         const uint32_t n = wave + 4 * i;
         if (n >= ntile) continue;
         const uint32_t tt = n / nv, t = tt * 32 + lq;
-        const float* v = r0 + 2 * sh.qk() + head * sh.vdim + n % nv * 32 + lq;
-#pragma unroll 2
-        for (uint32_t s = 0; s < 32 * (tt + 1); s += 16) acc[i] = mma32(column8(v, ld, s + 8 * lh, rows), load8(ps + t * LS + s + 8 * lh), acc[i]);
+#pragma unroll
+        for (uint32_t s = 0; s < 64; s += 16) {
+            if (s >= 32 * (tt + 1)) break;
+            acc[i] = mma32(i < EARLY ? vf[i < EARLY ? i : 0][s / 16] : values8(n, s), load8(ps + t * LS + s + 8 * lh), acc[i]);
+            __builtin_amdgcn_sched_barrier(0);
+        }
         float ss = 0.f;
 #pragma unroll
         for (int r = 0; r < 16; r++) ss = fmaf(acc[i][r], acc[i][r], ss);
@@ -399,7 +455,7 @@ void launch_linear_prompt(DType t, const LinearShape& sh, const LinearIo& io, ui
     static const hipError_t ok = hipFuncSetAttribute((const void*)linear_chunk_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
     (void)ok;
     fh::launch(linear_chunk_kernel, dim3(chunks, sh.heads), 256, chunk_lds(sh), s, sh, io.raw, io.w2, io.b2, M, decay, add, total);
-    fh::launch(linear_scan_kernel, dim3((uint32_t)((sh.state() / 2 + 255) / 256)), 256, 0, s, sh, chunks, total, add, io.state, io.base_pos);
+    fh::launch(linear_scan_kernel, dim3((uint32_t)((sh.state() + 255) / 256)), 256, 0, s, sh, chunks, total, add, io.state, io.base_pos);
     if (t == DType::BF16) output<__bf16>(sh, io, M, decay, add, norm, gate, out, ld_out, s);
     else output<float>(sh, io, M, decay, add, norm, gate, out, ld_out, s);
 }
