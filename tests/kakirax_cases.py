@@ -14,9 +14,9 @@ def cases(fh):
         "many_heads": (conf(128, 257, [att(40, 2, 32, 32, 96), gla(21, 32, 32, 96), att(17, 1, 64, 64, None)], embedding_scale=11.0), 16),
         # the largest heads; the largest rank of the decays' map
         "wide": (conf(160, 120, [gla(2, 256, 256, 100), att(2, 1, 256, 256, 100, scaling=(8.0, 1.0, 4.0, 64)), gla(1, 130, 200, None), att(3, 1, 130, 230, None)],
-                      embedding_scale=12.0, cap=50.0), 128),
+                      embedding_scale=12.5, cap=50.0), 128),
         # the variants between
-        "middle": (conf(192, 90, [gla(3, 64, 96, None), gla(2, 100, 128, 70), att(4, 2, 96, 32, None), att(2, 2, 128, 100, 40), att(4, 4, 64, 32, None), gla(2, 33, 70, None)],
+        "middle": (conf(192, 90, [gla(3, 64, 96, None), gla(2, 100, 128, 70), att(4, 2, 90, 40, None), att(2, 2, 128, 100, 40), att(4, 4, 64, 32, None), gla(2, 33, 70, None)],
                         embedding_scale=13.0), 33),
         # values that are 1 (or 2, where a pair has to be); eps keeps the norm of a lone value from being its mere sign
         "ones": (conf(33, 11, [gla(1, 1, 1, 1, tau=1.0), att(1, 1, 2, 1, 1), 0, att(2, 1, 3, 2, None, rot_dims=2)], embedding_scale=1.0, eps=0.5, cap=1.0), 1),
